@@ -213,7 +213,7 @@ class LLMEngine:
                 with open(path) as f:
                     conf = json.load(f)
                 # (designs that leave some sizes to the tensors get the checkpoint's header; HF checkpoints may be sharded)
-                shapes = safetensors_shapes(cfg.weights) if conf.get("architecture") == "Lemunex" else None
+                shapes = safetensors_shapes(cfg.weights) if conf.get("architecture") in ("Lemunex", "Beletar") else None
                 return from_config_json(conf, name=cfg.model, shapes=shapes)
         return resolve(cfg.model)
 

@@ -19,6 +19,10 @@ def model_class(cfg):
         from .dalalix import DalalixLM
 
         return DalalixLM
+    if family == "beletar":
+        from .beletar import BeletarLM
+
+        return BeletarLM
     if family == "llama":
         from .transformer import TransformerLM
 

@@ -67,9 +67,9 @@ class ModelConfig:
 # --------------------------------------------------------------------------------------------------
 @dataclass(frozen=True)
 class LatentMixerSpec:
-    """Attention through low-rank latents: queries via q_rank, keys / values via a cached kv_rank latent plus one
-    rotated key part of rot_dim shared by all heads.  ``kv_from``: the layer whose cache this layer attends
-    (it then has no down-projection of its own)."""
+    """Attention through low-rank latents: queries via q_rank (0: one projection, no latent), keys / values via a cached
+    kv_rank latent plus one rotated key part of rot_dim shared by all heads.  ``kv_from``: the layer whose cache this
+    layer attends (it then has no down-projection of its own)."""
     heads: int
     dim: int            # unrotated query / key dims per head
     rot_dim: int        # rotated dims per head (and of the shared key part)
@@ -83,6 +83,9 @@ class LatentMixerSpec:
     window: int = 0             # > 0: a position sees itself and the window - 1 positions before it; 0: all before it
     rot_half: bool = False      # rotary pairs dimension i with i + rot_dims / 2 instead of 2i with 2i + 1
     gate: bool = False          # head outputs times sigmoid(W_g h), element by element
+    head_gate: bool = False     # head h's output times sigmoid(W_g h)_h
+    sink: bool = False          # a learned per-head logit in the softmax's denominator (no key, no value)
+    rot_scaling: tuple | None = None   # (factor, original, fast, slow): blended rotary frequencies and a magnitude
 
 
 @dataclass(frozen=True)
@@ -1000,6 +1003,223 @@ SMALL_DALALIX = dalalix_stack("small-dalalix", 32768, 2048, "BPCC", heads=16, kv
                               expert_ff=1024, window=1024, mem_heads=8, mem_dim=128, mem_vdim=256, groups=4, keep=2,
                               buckets=65521, max_position=8192, bos_token_id=32000, eos_token_ids=(32001, 32002))
 
+# --------------------------------------------------------------------------------------------------
+# Beletar: pre-norm layers (layer norm with bias) listed one by one, a range of them run several times in a row with the
+# same weights (the embedding output added in front of every pass but the first, caches and states per pass); mixers: the
+# gated delta rule with one decay per head or one per key channel (short convolutions on q / k / v, unit-vector queries
+# and keys, gated per-head RMS norm), or causal latent attention with a sink and per-head output gates; silu-gated
+# feed-forward; logits through the embedding table.
+# --------------------------------------------------------------------------------------------------
+@dataclass(frozen=True)
+class DeltaSpec:
+    """Gated delta rule: S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q.  ``channel``: a decay per head and key
+    channel through a rank-``decay_rank`` projection and a sigmoid output gate through a rank-``gate_rank`` one; else a
+    decay per head and a silu output gate."""
+    heads: int
+    kv_heads: int                # query / key heads; query / key head j serves heads j * heads / kv_heads ..
+    dim: int
+    vdim: int
+    conv: int                    # taps of the causal per-channel convolutions
+    channel: bool = False
+    decay_rank: int = 0          # (both ranks from the checkpoint's tensor shapes)
+    gate_rank: int = 0
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+
+@dataclass(frozen=True)
+class SiluGluSpec:
+    ff: int
+
+
+@dataclass(frozen=True)
+class BeletarLayer:
+    type: str                    # "delta" | "channel_delta" | "latent_attention"
+    mixer: DeltaSpec | LatentMixerSpec
+    mlp: SiluGluSpec | None = None
+
+
+@dataclass(frozen=True)
+class LoopSpec:
+    """Layers start .. stop - 1 run ``times`` times in a row."""
+    start: int
+    stop: int
+    times: int
+
+
+@dataclass(frozen=True)
+class BeletarConfig:
+    family = "beletar"
+    name: str
+    vocab_size: int
+    hidden_size: int
+    layers: tuple
+    loop: LoopSpec | None = None
+    embed_scale: float = 1.0
+    norm_eps: float = 1e-6
+    max_position: int = 131072
+    bos_token_id: int = 1
+    eos_token_ids: tuple = (2,)
+    chat_format: str = "llama3"
+    tie_embeddings = True
+    rope_scaling = None
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def is_moe(self) -> bool:
+        return False
+
+    def layer_runs(self) -> list:
+        """The layers in the order they run: (layer, whether the embedding output is added in front of it).  Caches and
+        states belong to the entries of this list."""
+        n, lp = len(self.layers), self.loop
+        if lp is None:
+            return [(i, False) for i in range(n)]
+        out = [(i, False) for i in range(lp.start)]
+        for t in range(lp.times):
+            out += [(i, t > 0 and i == lp.start) for i in range(lp.start, lp.stop)]
+        return out + [(i, False) for i in range(lp.stop, n)]
+
+    def num_params(self) -> int:
+        from .weights import beletar_shapes
+
+        n = 0
+        for shape in beletar_shapes(self).values():
+            k = 1
+            for v in shape:
+                k *= v
+            n += k
+        return n
+
+    def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
+        return sum(self.layers[i].mixer.kv_rank + self.layers[i].mixer.rot_dim for i, _ in self.layer_runs()
+                   if self.layers[i].type == "latent_attention") * dtype_bytes
+
+    def state_bytes_per_seq(self, dtype_bytes: int = 2) -> int:
+        n = 0
+        for i, _ in self.layer_runs():
+            m = self.layers[i].mixer
+            if isinstance(m, DeltaSpec):
+                n += m.heads * m.dim * m.vdim * 4 + (m.conv - 1) * m.conv_channels * dtype_bytes
+        return n
+
+    def replace(self, **kw) -> "BeletarConfig":
+        return dataclasses.replace(self, **kw)
+
+
+def beletar_from_config(cfg: dict, name: str = "beletar", shapes: dict | None = None) -> BeletarConfig:
+    """config.json of a Beletar checkpoint: every size and constant is read here; a key this reader does not know means a
+    mechanism this code does not have, so it raises.  ``shapes`` (tensor name -> shape, the checkpoint's header) supplies
+    the sizes the configuration leaves to the tensors (the ranks of the decay and gate projections)."""
+    layers = []
+    for i, L in enumerate(cfg["layers"]):
+        kind, mixer, mlp = _take(L, f"layer {i}", "type", "mixer", optional=("mlp",))
+        if kind in ("delta", "channel_delta"):
+            conv, dim, heads, kvh, vdim = _take(mixer, f"layer {i} mixer", "conv", "dim", "heads", "kv_heads", "vdim")
+            ranks = (0, 0)
+            if kind == "channel_delta":
+                keys = (f"l{i}.mix.a1", f"l{i}.mix.g1")
+                if shapes is None or any(k not in shapes for k in keys):
+                    raise ValueError(f"layer {i}: the ranks of the decay and gate projections come from the shapes of "
+                                     f"{keys[0]} and {keys[1]}")
+                ranks = tuple(int(shapes[k][0]) for k in keys)
+            mix = DeltaSpec(int(heads), int(kvh), int(dim), int(vdim), int(conv), kind == "channel_delta", *ranks)
+            if mix.heads % mix.kv_heads or not 1 <= mix.conv <= 16:
+                raise ValueError(f"layer {i}: heads {heads} / kv_heads {kvh} / conv {conv} do not fit")
+        elif kind == "latent_attention":
+            dim, heads, r, rot, rd, scale, vdim = _take(mixer, f"layer {i} mixer", "dim", "heads", "kv_rank", "rot",
+                                                        "rot_dim", "scale", "vdim")
+            base, dims, scaling = _take(rot, f"layer {i} rot", "base", "dims", optional=("scaling",))
+            if scaling:
+                scaling = tuple(float(v) for v in _take(scaling, f"layer {i} rot.scaling", "factor", "original", "fast",
+                                                        "slow"))
+            mix = LatentMixerSpec(heads=int(heads), dim=int(dim), rot_dim=int(rd), vdim=int(vdim), kv_rank=int(r), q_rank=0,
+                                  rot_base=float(base), rot_dims=int(dims), scale=float(scale), head_gate=True, sink=True,
+                                  rot_scaling=scaling or None)
+            if mix.rot_dims > mix.rot_dim or mix.rot_dims % 2 or mix.rot_dim % 2:
+                raise ValueError(f"layer {i}: rot.dims {dims} / rot_dim {rd} do not fit")
+        else:
+            raise ValueError(f"layer {i}: unknown layer type {kind!r}")
+        if mlp is None:
+            ff = None
+        elif mlp.get("kind") == "dense":
+            (_, f) = _take(mlp, f"layer {i} mlp", "kind", "ff")
+            ff = SiluGluSpec(int(f))
+        else:
+            raise ValueError(f"layer {i}: unknown mlp kind {mlp.get('kind')!r}")
+        layers.append(BeletarLayer(kind, mix, ff))
+    vocab, width, norm, _, emb, loop, _, bos, eos = _take(
+        cfg, "config", "vocab", "width", "norm", "layers", "embedding",
+        optional=("loop", "architecture", "bos_token_id", "eos_token_ids"))
+    (eps,) = _take(norm, "norm", "eps")
+    (escale,) = _take(emb, "embedding", "scale")
+    if loop:
+        loop = LoopSpec(*(int(v) for v in _take(loop, "loop", "start", "stop", "times")))
+        if not 0 <= loop.start <= loop.stop <= len(layers) or loop.times < 1:
+            raise ValueError(f"loop {loop}: not a range of the {len(layers)} layers")
+    return BeletarConfig(name=name, vocab_size=int(vocab), hidden_size=int(width), layers=tuple(layers), loop=loop or None,
+                         embed_scale=float(escale), norm_eps=float(eps), bos_token_id=int(bos if bos is not None else 1),
+                         eos_token_ids=tuple(eos) if eos is not None else (2,))
+
+
+def beletar_to_config(c: BeletarConfig) -> dict:
+    """The config.json form of a BeletarConfig (exports, tests)."""
+    layers = []
+    for layer in c.layers:
+        m = layer.mixer
+        if layer.type == "latent_attention":
+            rot = {"base": m.rot_base, "dims": m.rot_dims}
+            if m.rot_scaling:
+                rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), m.rot_scaling))
+            md = {"dim": m.dim, "heads": m.heads, "kv_rank": m.kv_rank, "rot": rot, "rot_dim": m.rot_dim, "scale": m.scale,
+                  "vdim": m.vdim}
+        else:
+            md = {"conv": m.conv, "dim": m.dim, "heads": m.heads, "kv_heads": m.kv_heads, "vdim": m.vdim}
+        fd = None if layer.mlp is None else {"ff": layer.mlp.ff, "kind": "dense"}
+        layers.append({"mixer": md, "mlp": fd, "type": layer.type})
+    out = {"architecture": "Beletar", "embedding": {"scale": c.embed_scale}, "layers": layers, "norm": {"eps": c.norm_eps},
+           "vocab": c.vocab_size, "width": c.hidden_size}
+    if c.loop:
+        out["loop"] = {"start": c.loop.start, "stop": c.loop.stop, "times": c.loop.times}
+    return out
+
+
+def beletar_stack(name, vocab, width, pattern, heads, kv_heads, dim, vdim, ff, att_heads, att_dim=128, rot_dim=64,
+                  att_vdim=128, kv_rank=512, rank=128, conv=4, loop=None, embed_scale=1.0, scaling=None,
+                  **kw) -> BeletarConfig:
+    """A stack from a pattern string: "D" delta rule with head decays, "C" with channel decays, "L" latent attention; lower
+    case = no feed-forward.  ``loop`` = (start, stop, times)."""
+    layers = []
+    for ch in pattern:
+        if ch in "Dd":
+            kind, mix = "delta", DeltaSpec(heads, kv_heads, dim, vdim, conv)
+        elif ch in "Cc":
+            kind, mix = "channel_delta", DeltaSpec(heads, kv_heads, dim, vdim, conv, True, rank, rank)
+        elif ch in "Ll":
+            kind, mix = "latent_attention", LatentMixerSpec(
+                att_heads, att_dim, rot_dim, att_vdim, kv_rank, 0, 10000.0, rot_dim, (att_dim + rot_dim) ** -0.5,
+                head_gate=True, sink=True, rot_scaling=scaling)
+        else:
+            raise ValueError(f"pattern letter {ch!r}")
+        layers.append(BeletarLayer(kind, mix, SiluGluSpec(ff) if ch.isupper() else None))
+    return BeletarConfig(name=name, vocab_size=vocab, hidden_size=width, layers=tuple(layers),
+                         loop=LoopSpec(*loop) if loop else None, embed_scale=embed_scale, **kw)
+
+
+TINY_BELETAR = beletar_stack("tiny-beletar", 512, 128, "DCL", heads=4, kv_heads=2, dim=16, vdim=24, ff=192, att_heads=4,
+                             att_dim=16, rot_dim=8, att_vdim=20, kv_rank=48, rank=12, conv=3, loop=(0, 2, 2),
+                             embed_scale=4.0, scaling=(4.0, 256.0, 32.0, 1.0), max_position=2048, bos_token_id=500,
+                             eos_token_ids=(501, 502))
+# layer shapes of a mid-size model (benchmarks; random weights)
+SMALL_BELETAR = beletar_stack("small-beletar", 32768, 2048, "DCCL", heads=8, kv_heads=8, dim=128, vdim=256, ff=8192,
+                              att_heads=16, embed_scale=8.0, scaling=(4.0, 4096.0, 32.0, 1.0), max_position=8192,
+                              bos_token_id=32000, eos_token_ids=(32001, 32002))
+
 LLAMA31_SCALING = {
     "rope_type": "llama3",
     "factor": 8.0,
@@ -1042,7 +1262,8 @@ _REGISTRY = {
     c.name: c
     for c in (LLAMA3_8B, LLAMA31_8B, LLAMA3_70B, LLAMA31_70B, MIXTRAL_8X7B, TINY_LLAMA, TINY_MIXTRAL, SMALL_LLAMA,
               TINY_LLAMA_KV8, TINY_MIXTRAL_E8, TINY_BOZEVIK, SMALL_BOZEVIK, SMALL_BOZEVIK_MOE, TINY_LEMUNEX,
-              SMALL_LEMUNEX, SMALL_LEMUNEX_MOE, TINY_KOMAZEN, SMALL_KOMAZEN, TINY_DALALIX, SMALL_DALALIX)
+              SMALL_LEMUNEX, SMALL_LEMUNEX_MOE, TINY_KOMAZEN, SMALL_KOMAZEN, TINY_DALALIX, SMALL_DALALIX,
+              TINY_BELETAR, SMALL_BELETAR)
 }
 _ALIASES = {
     "llama3": "llama3:8b",
@@ -1075,8 +1296,8 @@ def known_models() -> list[str]:
 
 def from_config_json(cfg: dict, name: str = "hf", shapes: dict | None = None):
     """The model configuration of a checkpoint directory's config.json: the design is chosen by its
-    ``architecture`` key (Bozevik, Lemunex, Komazen, Dalalix), otherwise the HuggingFace Llama / Mixtral keys.  ``shapes``: the
-    checkpoint's tensor shapes, for designs that leave some sizes to them."""
+    ``architecture`` key (Bozevik, Lemunex, Komazen, Dalalix, Beletar), otherwise the HuggingFace Llama / Mixtral keys.  ``shapes``:
+    the checkpoint's tensor shapes, for designs that leave some sizes to them."""
     if cfg.get("architecture") == "Bozevik":
         return bozevik_from_config(cfg, name)
     if cfg.get("architecture") == "Lemunex":
@@ -1085,6 +1306,8 @@ def from_config_json(cfg: dict, name: str = "hf", shapes: dict | None = None):
         return komazen_from_config(cfg, name)
     if cfg.get("architecture") == "Dalalix":
         return dalalix_from_config(cfg, name)
+    if cfg.get("architecture") == "Beletar":
+        return beletar_from_config(cfg, name, shapes)
     return from_hf_config(cfg, name)
 
 

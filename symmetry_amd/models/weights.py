@@ -186,6 +186,8 @@ def random_weights(cfg: ModelConfig, shard: ShardSpec | None = None, device="cpu
         return komazen_random_weights(cfg, shard, device, dtype, seed)
     if getattr(cfg, "family", "llama") == "dalalix":
         return dalalix_random_weights(cfg, shard, device, dtype, seed)
+    if getattr(cfg, "family", "llama") == "beletar":
+        return beletar_random_weights(cfg, shard, device, dtype, seed)
     shard.validate(cfg)
     shapes = full_shapes(cfg)
     tensors = {}
@@ -246,6 +248,8 @@ def load_hf_weights(path: str, cfg: ModelConfig, shard: ShardSpec | None = None,
         return load_komazen_weights(path, cfg, shard, device, dtype)
     if getattr(cfg, "family", "llama") == "dalalix":
         return load_dalalix_weights(path, cfg, shard, device, dtype)
+    if getattr(cfg, "family", "llama") == "beletar":
+        return load_beletar_weights(path, cfg, shard, device, dtype)
     shard.validate(cfg)
     wmap = _hf_index(path)
     handles = {}
@@ -788,5 +792,113 @@ def save_dalalix_checkpoint(weights: ModelWeights, path: str) -> None:
     os.makedirs(path, exist_ok=True)
     with open(os.path.join(path, "config.json"), "w") as f:
         json.dump(dalalix_to_config(weights.cfg), f, indent=1)
+    save_file({k: v.detach().to(torch.bfloat16).contiguous().cpu() for k, v in weights.tensors.items()},
+              os.path.join(path, "model.safetensors"))
+
+
+# --------------------------------------------------------------------------------------------------
+# Beletar checkpoints: tensors keep the checkpoint's names (embed, l<i>.norm1, l<i>.norm1.b, l<i>.mix.q, l<i>.mix.q.conv,
+# l<i>.mix.A_log, l<i>.mix.dkv, l<i>.mlp.gate, ..., final.norm, final.norm.b); a layer that runs several times has its
+# tensors once.  models/beletar.py fuses what its GEMMs read.
+# --------------------------------------------------------------------------------------------------
+def beletar_shapes(cfg, optional: set | None = None) -> dict:
+    """Tensor name -> shape.  ``optional`` (a set) receives the names a checkpoint may carry without this code reading
+    them: the second norm of a layer that has no feed-forward."""
+    d = cfg.hidden_size
+    shapes = {"embed": (cfg.vocab_size, d), "final.norm": (d,), "final.norm.b": (d,)}
+    for i, layer in enumerate(cfg.layers):
+        p, m, q = f"l{i}.", layer.mixer, f"l{i}.mix."
+        shapes[p + "norm1"] = shapes[p + "norm1.b"] = (d,)
+        if layer.type == "latent_attention":
+            shapes[q + "q"] = (m.heads * (m.dim + m.rot_dim), d)
+            shapes[q + "dkv"], shapes[q + "dkv.norm"] = (m.kv_rank + m.rot_dim, d), (m.kv_rank,)
+            shapes[q + "uk"], shapes[q + "uv"] = (m.heads * m.dim, m.kv_rank), (m.heads * m.vdim, m.kv_rank)
+            shapes[q + "sink"], shapes[q + "g"] = (m.heads,), (m.heads, d)
+        else:
+            for nm, rows in (("q", m.kv_heads * m.dim), ("k", m.kv_heads * m.dim), ("v", m.heads * m.vdim)):
+                shapes[q + nm], shapes[f"{q}{nm}.conv"] = (rows, d), (rows, m.conv)
+            shapes[q + "b"], shapes[q + "A_log"], shapes[q + "norm"] = (m.heads, d), (m.heads,), (m.vdim,)
+            if m.channel:
+                shapes[q + "a1"], shapes[q + "a2"] = (m.decay_rank, d), (m.heads * m.dim, m.decay_rank)
+                shapes[q + "dt_bias"] = (m.heads * m.dim,)
+                shapes[q + "g1"], shapes[q + "g2"] = (m.gate_rank, d), (m.heads * m.vdim, m.gate_rank)
+            else:
+                shapes[q + "a"], shapes[q + "dt_bias"] = (m.heads, d), (m.heads,)
+                shapes[q + "g"] = (m.heads * m.vdim, d)
+        shapes[q + "o"] = (d, m.heads * m.vdim)
+        if layer.mlp is not None:
+            f = layer.mlp.ff
+            shapes[p + "norm2"] = shapes[p + "norm2.b"] = (d,)
+            shapes[p + "mlp.gate"], shapes[p + "mlp.up"], shapes[p + "mlp.down"] = (f, d), (f, d), (d, f)
+        elif optional is not None:
+            optional.update((p + "norm2", p + "norm2.b"))
+    return shapes
+
+
+def beletar_random_weights(cfg, shard: ShardSpec | None = None, device="cpu", dtype=torch.bfloat16,
+                           seed: int = 0) -> ModelWeights:
+    """Random init (benchmarks, tests): matrices N(0, (1.28 / sqrt(fan_in))^2); norm weights around one; norm biases, sinks
+    and convolution taps nonzero; decays from a few to a few hundred tokens -- all away from the values at which a dropped
+    parameter would not show."""
+    shard = shard or ShardSpec()
+    if shard.tp_size > 1 or shard.ep_size > 1:
+        raise NotImplementedError("Beletar runs on one GPU per replica (its tensors are not sharded)")
+    tensors = {}
+    for name, shape in beletar_shapes(cfg).items():
+        g = torch.Generator().manual_seed(_seed(seed, name))
+        leaf = name.rsplit(".", 1)[-1]
+        if leaf in ("norm", "norm1", "norm2"):
+            t = 0.75 + 0.5 * torch.rand(shape, generator=g)
+        elif name.endswith("norm.b") or name.endswith("norm1.b") or name.endswith("norm2.b"):
+            t = 0.2 * torch.randn(shape, generator=g)
+        elif leaf == "A_log":
+            t = torch.log(0.02 + 0.5 * torch.rand(shape, generator=g))
+        elif leaf == "dt_bias":
+            t = -2.0 + torch.rand(shape, generator=g)
+        elif leaf == "sink":
+            t = torch.randn(shape, generator=g)
+        elif leaf == "conv":
+            t = torch.randn(shape, generator=g) * shape[1] ** -0.5
+        else:      # (the embedding table is the output head too: its rows are scaled like any matrix of this width)
+            tensors[name] = _randn(shape, _seed(seed, name), device, dtype, _std("head" if name == "embed" else name, shape))
+            continue
+        tensors[name] = t.to(dtype).to(device)
+    return ModelWeights(cfg, shard, tensors)
+
+
+def load_beletar_weights(path: str, cfg, shard: ShardSpec | None = None, device="cpu",
+                         dtype=torch.bfloat16) -> ModelWeights:
+    """model.safetensors of a Beletar checkpoint directory; every tensor the configuration implies must be there with the
+    implied shape, and no other.  Tensors stay in the file's precision (the model converts what it fuses)."""
+    from safetensors import safe_open
+
+    shard = shard or ShardSpec()
+    if shard.tp_size > 1 or shard.ep_size > 1:
+        raise NotImplementedError("Beletar runs on one GPU per replica (its tensors are not sharded)")
+    optional: set = set()
+    shapes = beletar_shapes(cfg, optional)
+    tensors = {}
+    with safe_open(os.path.join(path, "model.safetensors"), framework="pt") as f:
+        names = set(f.keys())
+        missing, extra = sorted(set(shapes) - names), sorted(names - set(shapes) - optional)
+        if missing or extra:
+            raise ValueError(f"checkpoint does not fit its config: missing {missing[:4]}, unexpected {extra[:4]}")
+        for name, shape in shapes.items():
+            t = f.get_tensor(name)
+            if tuple(t.shape) != tuple(shape):
+                raise ValueError(f"{name}: shape {tuple(t.shape)}, the config implies {tuple(shape)}")
+            tensors[name] = t.to(device)
+    return ModelWeights(cfg, shard, tensors)
+
+
+def save_beletar_checkpoint(weights: ModelWeights, path: str) -> None:
+    """config.json + model.safetensors (bf16) of a Beletar model, in the form the loader reads."""
+    from safetensors.torch import save_file
+
+    from .config import beletar_to_config
+
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(beletar_to_config(weights.cfg), f, indent=1)
     save_file({k: v.detach().to(torch.bfloat16).contiguous().cpu() for k, v in weights.tensors.items()},
               os.path.join(path, "model.safetensors"))

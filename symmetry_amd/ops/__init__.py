@@ -536,6 +536,15 @@ def linear(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None) ->
     return torch.matmul(x, w.t(), out=out)
 
 
+def linear_f32(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """out (fp32) = x @ w.T with the library GEMM's fp32 accumulator left unrounded; x, w bf16 or fp32."""
+    if x.dtype == torch.float32:
+        return torch.mm(x, w.t(), out=out)
+    if x.device.type == "cpu":
+        return out.copy_(x.float() @ w.float().t())
+    return torch.mm(x, w.t(), out_dtype=torch.float32, out=out)
+
+
 def lib_splits(M: int, N: int, K: int) -> int:
     """k split of a library prefill GEMM run as one strided-batched GEMM into fp32 slabs (linear_splitk).
     The narrow projections (N <= 8192) of 257..768-token prefills (and long-K ones up to 1536) leave most CUs
@@ -628,7 +637,7 @@ def latent_prep(z, q_rank, kv_rank, rot, wq, wkv, eps, positions, slots, rope, c
     """z [T, q_rank (+ kv_rank + rot)] (a view: further columns may follow in its rows) -> cq = rms_norm(z[:, :q_rank]) *
     wq; with a kv part (kv_rank > 0) the token's cache row (slot >= 0) becomes [rms_norm(z kv part) * wkv | rotary(z rot
     part)].  ``half_dims`` = 0: rotary pairs (2i, 2i + 1); > 0: the half layout, entry i < half_dims / 2 paired with
-    i + half_dims / 2 and the entries past half_dims passing."""
+    i + half_dims / 2 and the entries past half_dims passing.  ``q_rank`` = 0: no query latent (wq and cq None)."""
     if _gpu(z):
         return _lat().latent_prep(z, int(q_rank), int(kv_rank), int(rot), wq, wkv, float(eps), positions, slots, rope,
                                   cq, cache, int(half_dims))
@@ -653,7 +662,7 @@ LATENT_ATTN_IMPL = 1 if os.environ.get("SYMMETRY_LATENT_ATTN", "mfma") == "wave"
 
 
 def latent_attn(q, cache, block_tables, row_seq, positions, scale, kv_rank, out, part_o=None, part_ml=None,
-                tiles=None, cu_q=None, impl=None, window=0):
+                tiles=None, cu_q=None, impl=None, window=0, sink=None, gate=None):
     """Causal softmax attention of q [T, H, Dk] over the paged latent cache [NB, BS, Dk]: keys are whole cache rows,
     values their first kv_rank entries; row r sees keys 0..positions[r] of sequence row_seq[r].  ``part_o``
     [T, H, parts, kv_rank] / ``part_ml`` [T, H, parts, 2]: split-KV scratch (decode steps: ``parts`` equal partitions of
@@ -663,11 +672,13 @@ def latent_attn(q, cache, block_tables, row_seq, positions, scale, kv_rank, out,
     (decode steps).  Other shapes, fp32 and ``impl=1`` run the one-wave-per-(row, head) kernel.  Returns the
     implementation used (0 MFMA, 1 wave).  ``window`` > 0: row r sees only the keys positions[r] - window + 1 ..
     positions[r], and the split-KV partitions cover that range (count them with ``latent_attn_parts(rows, min(span,
-    window))``)."""
+    window))``).  ``sink`` [H] fp32: the softmax's denominator of head h also holds exp(sink[h]) (a logit without a key or a
+    value, not scaled).  ``gate`` [T, H] (a view): head outputs are multiplied by sigmoid(gate)."""
     if _gpu(q):
         return _lat().latent_attn(q, cache, block_tables, row_seq, positions, float(scale), int(kv_rank), out, part_o,
-                                  part_ml, tiles, cu_q, LATENT_ATTN_IMPL if impl is None else int(impl), int(window))
-    reference.latent_attn(q, cache, block_tables, row_seq, positions, scale, kv_rank, out, window)
+                                  part_ml, tiles, cu_q, LATENT_ATTN_IMPL if impl is None else int(impl), int(window), sink,
+                                  gate)
+    reference.latent_attn(q, cache, block_tables, row_seq, positions, scale, kv_rank, out, window, sink, gate)
     return 1
 
 
@@ -816,12 +827,12 @@ def memory_norm_gate(y, m, gate, w, eps, out):
     return reference.memory_norm_gate(y, m, gate, w, eps, out)
 
 
-def gated_group_norm(y, gate, w, eps, group, gate_first, out):
-    """y fp32 [T, C], gate [T, C] (view): s = silu(gate); gate_first: out = rms_group(y s) w, else rms_group(y) w s;
-    rms over groups of ``group`` columns; w [len] repeats over the columns (C % len == 0)."""
+def gated_group_norm(y, gate, w, eps, group, gate_first, out, sigmoid=False):
+    """y fp32 [T, C], gate [T, C] (view): s = silu(gate), or sigmoid(gate); gate_first: out = rms_group(y s) w, else
+    rms_group(y) w s; rms over groups of ``group`` columns; w [len] repeats over the columns (C % len == 0)."""
     if _gpu(y):
-        return _hyb().gated_group_norm(y, gate, w, float(eps), int(group), bool(gate_first), out)
-    return reference.gated_group_norm(y, gate, w, eps, group, gate_first, out)
+        return _hyb().gated_group_norm(y, gate, w, float(eps), int(group), bool(gate_first), out, bool(sigmoid))
+    return reference.gated_group_norm(y, gate, w, eps, group, gate_first, out, sigmoid)
 
 
 def causal_conv_silu(xin, w, b, state, cu_q, row_seq, prev_row, runs, out):
@@ -1017,3 +1028,49 @@ def logit_softcap(logits, cap):
     if _gpu(logits):
         return _hyb().logit_softcap(logits, float(cap))
     return reference.logit_softcap(logits, cap)
+
+
+def residual_layer_norm(x, a=None, b=None, w=None, bias=None, eps=0.0, rows=None, out=None, base=None):
+    """fp32 stream x [T, d]: x = base + a + b (``base`` defaults to x itself; a and b [T, d] optional, bf16 or fp32), and
+    with ``out``: out[i] = layer_norm(x[rows ? rows[i] : i]) * w + bias (variance = mean of squared deviations), the next
+    sublayer's input from the same pass.  ``rows`` (a gather in front of the output head) comes without a sum."""
+    if _gpu(x):
+        return _hyb().residual_layer_norm(x, base, a, b, w, bias, float(eps), rows, out)
+    return reference.residual_layer_norm(x, a, b, w, bias, eps, rows, out, base)
+
+
+def conv_silu_qkv(z, w, state, cu_q, row_seq, prev_row, runs, G, N, H, P, q_scale, unit_eps, q_out, k_out, v_out,
+                  save_slot=None):
+    """z [T, G N | G N | H P] (a view) = q | k | v through the causal per-channel convolution w [C, taps] over every run
+    (inputs before a run from state[slot] [taps - 1, C] where prev_row[first] <= -2, else zero), then silu; q and k heads
+    (N entries) become unit vectors y / sqrt(sum y^2 + unit_eps), q also times q_scale -> q_out, k_out fp32 [T, G, N]; v ->
+    v_out [T, H, P].  ``save_slot`` with cu_q None (every row its own run): the launch moves the row's carried taps on
+    itself; otherwise conv_state_update follows."""
+    if _gpu(z):
+        return _hyb().conv_silu_qkv(z, w, state, cu_q, row_seq if cu_q is not None else None, prev_row, save_slot, int(runs),
+                                    int(G), int(N), int(H), int(P), float(q_scale), float(unit_eps), q_out, k_out, v_out)
+    reference.conv_silu_qkv(z, w, state, cu_q, prev_row, runs, G, N, H, P, q_scale, unit_eps, q_out, k_out, v_out)
+    if save_slot is not None and state.shape[1]:
+        reference.conv_state_update(z, state, cu_q, prev_row, save_slot, runs)
+
+
+DELTA_CHUNK = 32            # tokens per chunk of delta_rule's chunked form (csrc/kernels/delta_rule.hip)
+DELTA_IMPL = 1 if os.environ.get("SYMMETRY_DELTA_RULE", "auto") == "serial" else 0  # A/B: the token-by-token kernel
+
+
+def delta_rule(channel, q, k, v, dz, dt_bias, A_log, bz, state, cu_q, prev_row, save_slot, runs, out, tiles=None, ws=None,
+               impl=None):
+    """Gated delta rule per head h over every run of rows (cu_q[i] .. cu_q[i + 1]; cu_q None: every row its own run), state
+    S [N, P] fp32:  S <- g_t S;  u = beta_t (v_t - S^T k_t);  S <- S + k_t u^T;  out_t = S^T q_t.
+    beta = sigmoid(bz[:, h]); log g = -exp(A_log[h]) softplus(dz + dt_bias), one per head (dz, bz fp32 [T, H]) or with
+    ``channel`` one per head and key channel (dz fp32 [T, H N]).  q, k fp32 [T, G, N]: head h reads h // (H / G); v [T, H, P]
+    bf16 or fp32.  A run starts from state[slot] if prev_row[first] <= -2 (slot = -(v + 2)), else from zero; it ends in
+    state[save_slot[last]] (>= 0).  out fp32 [T, H, P].
+    ``tiles`` [n, 2] (sequence, first row of a 64-row tile within the run) + ``ws`` (fp32 scratch of delta_ws_elems):
+    prompt steps take the chunked form (N <= 256), else and with ``impl=1`` the token-by-token kernel.  Returns the
+    implementation used (0 chunked, 1 token by token)."""
+    if _gpu(out):
+        return _hyb().delta_rule(bool(channel), q, k, v, dz, dt_bias, A_log, bz, state, cu_q, prev_row, save_slot, int(runs),
+                                 out, tiles, ws, DELTA_IMPL if impl is None else int(impl))
+    reference.delta_rule(channel, q, k, v, dz, dt_bias, A_log, bz, state, cu_q, prev_row, save_slot, runs, out)
+    return 1

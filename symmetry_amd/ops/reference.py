@@ -633,8 +633,9 @@ def _rot(v, cs, half_dims):
 def latent_prep(z, q_rank, kv_rank, rot, wq, wkv, eps, positions, slots, rope, cq, cache, half_dims=0) -> None:
     T = z.shape[0]
     zf = z.float()
-    q = zf[:, :q_rank]
-    cq.copy_((q / torch.sqrt((q * q).mean(-1, keepdim=True) + eps) * wq.float()).to(cq.dtype))
+    if q_rank:
+        q = zf[:, :q_rank]
+        cq.copy_((q / torch.sqrt((q * q).mean(-1, keepdim=True) + eps) * wq.float()).to(cq.dtype))
     if not kv_rank:
         return
     c = zf[:, q_rank:q_rank + kv_rank]
@@ -651,7 +652,8 @@ def rope_pairs(src, dst, positions, rope, half_dims=0) -> None:
     dst.copy_(_rot(src.float(), rope[positions[:T].long()][:, None], half_dims).to(dst.dtype))
 
 
-def latent_attn(q, cache, block_tables, row_seq, positions, scale, kv_rank, out, window=0) -> None:
+def latent_attn(q, cache, block_tables, row_seq, positions, scale, kv_rank, out, window=0, sink=None,
+                gate=None) -> None:
     T, H, Dk = q.shape
     BS = cache.shape[1]
     o = out.view(T, H, kv_rank)
@@ -661,8 +663,14 @@ def latent_attn(q, cache, block_tables, row_seq, positions, scale, kv_rank, out,
         idx = torch.arange(max(0, n - window) if window > 0 else 0, n)
         rows = cache[bt[idx // BS], idx % BS].float()          # [n, Dk]
         s = (q[r].float() @ rows.t()) * scale                   # [H, n]
-        p = torch.softmax(s, -1)
-        o[r] = (p @ rows[:, :kv_rank]).to(out.dtype)
+        if sink is not None:     # one more logit in the denominator, without a value
+            p = torch.softmax(torch.cat([s, sink.float()[:, None]], -1), -1)[:, :-1]
+        else:
+            p = torch.softmax(s, -1)
+        y = p @ rows[:, :kv_rank]
+        if gate is not None:
+            y = y * torch.sigmoid(gate[r].float())[:, None]
+        o[r] = y.to(out.dtype)
 
 
 def clamped_glu(gu, limit, alpha, out) -> None:
@@ -889,10 +897,10 @@ def memory_norm_gate(y, m, gate, w, eps, out) -> None:
     out.copy_((o * w.float() * torch.sigmoid(gate.float())).to(out.dtype))
 
 
-def gated_group_norm(y, gate, w, eps, group, gate_first, out) -> None:
+def gated_group_norm(y, gate, w, eps, group, gate_first, out, sigmoid=False) -> None:
     T, C = y.shape
     g = gate.float()
-    g = g * torch.sigmoid(g)
+    g = torch.sigmoid(g) if sigmoid else g * torch.sigmoid(g)
     v = y * g if gate_first else y
     v = _unit_rms(v.view(T, C // group, group), eps).reshape(T, C)
     v = v * w.float().repeat(C // w.numel())
@@ -1084,3 +1092,55 @@ def conv_qkv_cache(z, w, state, cu_q, prev_row, runs, H, G, dk, dv, v_eps, slots
 
 def logit_softcap(logits, cap) -> None:
     logits.copy_(cap * torch.tanh(logits / cap))
+
+
+# ---- pre-norm stream with biased layer norms, gated delta rule (the Beletar layers) -----------------------------
+def residual_layer_norm(x, a, b, w, bias, eps, rows, out, base=None) -> None:
+    v = x if base is None else base
+    for t in (a, b):
+        if t is not None:
+            v = v + t.float().view_as(x)
+    if v is not x:
+        x.copy_(v)
+    if out is not None:
+        n = out.shape[0]
+        r = x[rows[:n].long()] if rows is not None else x[:n]
+        out.copy_((_ln(r, w, eps) + bias.float()).to(out.dtype))
+
+
+def conv_silu_qkv(z, w, state, cu_q, prev_row, runs, G, N, H, P, q_scale, unit_eps, q_out, k_out, v_out) -> None:
+    T, C = z.shape[0], w.shape[0]
+    y = torch.empty(T, C)
+    causal_conv_silu(z[:, :C], w, torch.zeros(C), state, cu_q, prev_row, runs, y)
+
+    def unit(t):
+        return t / torch.sqrt((t * t).sum(-1, keepdim=True) + unit_eps)
+
+    q_out.copy_(unit(y[:, :G * N].view(T, G, N)) * q_scale)
+    k_out.copy_(unit(y[:, G * N:2 * G * N].view(T, G, N)))
+    v_out.copy_(y[:, 2 * G * N:].view(T, H, P).to(v_out.dtype))
+
+
+def delta_rule(channel, q, k, v, dz, dt_bias, A_log, bz, state, cu_q, prev_row, save_slot, runs, out) -> None:
+    """S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q per head over every run of rows."""
+    T, G, N = q.shape
+    H, P = v.shape[1:]
+    grp = torch.arange(H) // (H // G)
+    z = dz.float().reshape(T, H, -1) + dt_bias.float().view(H, -1)
+    g = torch.exp(-torch.exp(A_log.float())[None, :, None] * torch.nn.functional.softplus(z, threshold=1e9)).expand(T, H, N)
+    beta = torch.sigmoid(bz.float())
+    o = out.view(T, H, P)
+    for s0, s1 in _runs(T, cu_q, runs):
+        if s1 <= s0:
+            continue
+        pr = int(prev_row[s0])
+        S = state[-(pr + 2)].clone() if pr <= -2 else torch.zeros(H, N, P)
+        for t in range(s0, s1):
+            S = g[t][:, :, None] * S
+            kt = k[t, grp]
+            u = beta[t][:, None] * (v[t].float() - torch.einsum("hnp,hn->hp", S, kt))
+            S = S + kt[:, :, None] * u[:, None, :]
+            o[t] = torch.einsum("hnp,hn->hp", S, q[t, grp])
+        sv = int(save_slot[s1 - 1])
+        if sv >= 0:
+            state[sv] = S
