@@ -1,5 +1,5 @@
-// TORCH_LIBRARY registration of the kernels in hybrid_rows.hip, stream_rows.hip, window_attention.hip and decay_scan.hip, plus the
-// expert-segment kernels of glu_moe.hip that the routed feed-forward shares (symmetry_amd/_C_hybrid.so, namespace
+// TORCH_LIBRARY registration of the kernels in hybrid_rows.hip, stream_rows.hip, window_attention.hip, decay_scan.hip and
+// delta_rule.hip, plus the expert-segment kernels of glu_moe.hip that the routed feed-forward shares (symmetry_amd/_C_hybrid.so, namespace
 // symmetry_amd_hybrid).
 //
 // Out-parameter style like the other kernel libraries: the caller pre-allocates, nothing is allocated here, every
@@ -303,7 +303,7 @@ void decay_scan(int64_t mode, const Tensor& q, const Tensor& k, const Tensor& v,
 }
 
 void gated_group_norm(const Tensor& y, const Tensor& gate, const Tensor& w, double eps, int64_t group, bool gate_first,
-                      Tensor& out) {
+                      Tensor& out, bool sigmoid) {
   const int f32 = act(out, "out");
   dtype(y, at::kFloat, "y");
   dtype(w, at::kFloat, "w");
@@ -313,7 +313,7 @@ void gated_group_norm(const Tensor& y, const Tensor& gate, const Tensor& w, doub
   TORCH_CHECK(group > 0 && C % group == 0 && w.numel() > 0 && C % w.numel() == 0 && out.numel() == T * C &&
                   C / group <= 65535, "gated_group_norm: shapes");
   launch_gated_group_norm(ptr<float>(y), gate.data_ptr(), ldg, ptr<float>(w), (int)w.numel(), (float)eps, (int)group,
-                          gate_first ? 1 : 0, out.data_ptr(), (int)T, (int)C, f32, cur_stream(y));
+                          gate_first ? 1 : 0, sigmoid ? 1 : 0, out.data_ptr(), (int)T, (int)C, f32, cur_stream(y));
 }
 
 ConvArgs conv_args(const Tensor& xin, const OptTensor& w, const OptTensor& b, Tensor& state, const OptTensor& cu_q,
@@ -774,6 +774,160 @@ void logit_softcap(Tensor& logits, double cap) {
   launch_logit_softcap(ptr<float>(logits), logits.numel(), (float)cap, cur_stream(logits));
 }
 
+void residual_layer_norm(Tensor& x, const OptTensor& base, const OptTensor& a, const OptTensor& b, const OptTensor& w,
+                         const OptTensor& bias, double eps, const OptTensor& rows, OptTensor out) {
+  dtype(x, at::kFloat, "x");
+  TORCH_CHECK(x.dim() == 2, "residual_layer_norm: x [T, d]");
+  const int64_t T = x.size(0), d = x.size(1);
+  ResidualLnArgs r{};
+  r.x = ptr<float>(x);
+  r.n = (int)T;
+  r.d = (int)d;
+  r.eps = (float)eps;
+  if (base.has_value()) {
+    dtype(*base, at::kFloat, "base");
+    TORCH_CHECK(base->numel() == T * d, "residual_layer_norm: base shape");
+    r.base = ptr<float>(*base);
+  }
+  if (a.has_value()) {
+    r.a_f32 = act(*a, "a");
+    TORCH_CHECK(a->numel() == T * d, "residual_layer_norm: a shape");
+    r.a = a->data_ptr();
+  }
+  if (b.has_value()) {
+    r.b_f32 = act(*b, "b");
+    TORCH_CHECK(b->numel() == T * d, "residual_layer_norm: b shape");
+    r.b = b->data_ptr();
+  }
+  int f32 = 0;
+  if (out.has_value()) {
+    f32 = act(*out, "out");
+    TORCH_CHECK(w.has_value() && bias.has_value(), "residual_layer_norm: out without w and bias");
+    dtype(*w, at::kFloat, "w");
+    dtype(*bias, at::kFloat, "bias");
+    TORCH_CHECK(out->dim() == 2 && out->size(1) == d && w->numel() == d && bias->numel() == d,
+                "residual_layer_norm: out / w / bias shape");
+    r.out = out->data_ptr();
+    r.w = ptr<float>(*w);
+    r.bias = ptr<float>(*bias);
+    if (rows.has_value()) {
+      TORCH_CHECK(!base.has_value() && !a.has_value() && !b.has_value(), "residual_layer_norm: gathered rows take no sum");
+      dtype(*rows, at::kLong, "rows");
+      TORCH_CHECK(rows->numel() >= out->size(0), "residual_layer_norm: rows too short");
+      r.rows = ptr<long long>(*rows);
+      r.n = (int)out->size(0);
+    } else {
+      const bool sum = base.has_value() || a.has_value() || b.has_value();
+      TORCH_CHECK(sum ? out->size(0) == T : out->size(0) <= T, "residual_layer_norm: out rows");
+      r.n = (int)out->size(0);
+    }
+  } else {
+    TORCH_CHECK(!rows.has_value(), "residual_layer_norm: rows without out");
+  }
+  launch_residual_layer_norm(r, f32, cur_stream(x));
+}
+
+void conv_silu_qkv(const Tensor& z, const Tensor& w, Tensor& state, const OptTensor& cu_q, const OptTensor& row_seq,
+                   const Tensor& prev_row, const OptTensor& save_slot, int64_t runs, int64_t G, int64_t N, int64_t H,
+                   int64_t P, double q_scale, double unit_eps, Tensor& q_out, Tensor& k_out, Tensor& v_out) {
+  const int f32 = act(w, "w");
+  TORCH_CHECK(z.dim() == 2 && w.dim() == 2 && state.dim() == 3, "conv_silu_qkv: z [T, C], w [C, taps], state [slots, taps - 1, C]");
+  const int64_t T = z.size(0), C = 2 * G * N + H * P, taps = w.size(1);
+  TORCH_CHECK(G > 0 && H > 0 && N > 0 && P > 0 && N <= 512 && P <= 512 && taps >= 1 && taps <= 16 && w.size(0) == C,
+              "conv_silu_qkv: sizes (heads up to 512 wide, at most 16 taps)");
+  ConvSiluArgs a{};
+  a.ldz = view2(z, f32, T, C, "z");
+  same_act(state, f32, "state");
+  same_act(v_out, f32, "v_out");
+  dtype(q_out, at::kFloat, "q_out");
+  dtype(k_out, at::kFloat, "k_out");
+  dtype(prev_row, at::kInt, "prev_row");
+  TORCH_CHECK(state.size(1) == taps - 1 && state.size(2) == C && q_out.numel() == T * G * N && k_out.numel() == T * G * N &&
+                  v_out.numel() == T * H * P && prev_row.numel() >= T && 2 * G + H <= 65535, "conv_silu_qkv: shapes");
+  if (cu_q.has_value()) {
+    TORCH_CHECK(row_seq.has_value(), "conv_silu_qkv: cu_q without row_seq");
+    dtype(*cu_q, at::kInt, "cu_q");
+    dtype(*row_seq, at::kInt, "row_seq");
+    TORCH_CHECK(cu_q->numel() >= runs + 1 && row_seq->numel() >= T, "conv_silu_qkv: run metadata");
+    a.cu_q = ptr<int>(*cu_q);
+    a.row_seq = ptr<int>(*row_seq);
+  }
+  if (save_slot.has_value()) {
+    TORCH_CHECK(!cu_q.has_value(), "conv_silu_qkv: save_slot is for rows that are runs of their own");
+    dtype(*save_slot, at::kInt, "save_slot");
+    TORCH_CHECK(save_slot->numel() >= T, "conv_silu_qkv: save_slot too short");
+    a.save_slot = ptr<int>(*save_slot);
+  }
+  a.z = z.data_ptr();
+  a.w = w.data_ptr();
+  a.state = state.data_ptr();
+  a.state_stride = state.stride(0);
+  a.prev_row = ptr<int>(prev_row);
+  a.q_out = ptr<float>(q_out);
+  a.k_out = ptr<float>(k_out);
+  a.v_out = v_out.data_ptr();
+  a.q_scale = (float)q_scale;
+  a.eps = (float)unit_eps;
+  a.T = (int)T, a.C = (int)C, a.taps = (int)taps, a.G = (int)G, a.N = (int)N, a.H = (int)H, a.P = (int)P;
+  launch_conv_silu_qkv(a, f32, cur_stream(z));
+}
+
+int64_t delta_rule(bool channel, const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& dz, const Tensor& dt_bias,
+                   const Tensor& A_log, const Tensor& bz, Tensor& state, const OptTensor& cu_q, const Tensor& prev_row,
+                   const Tensor& save_slot, int64_t runs, Tensor& out, const OptTensor& tiles, const OptTensor& ws,
+                   int64_t impl) {
+  const int f32 = act(v, "v");
+  dtype(q, at::kFloat, "q");
+  dtype(k, at::kFloat, "k");
+  dtype(out, at::kFloat, "out");
+  dtype(state, at::kFloat, "state");
+  dtype(dt_bias, at::kFloat, "dt_bias");
+  dtype(A_log, at::kFloat, "A_log");
+  dtype(prev_row, at::kInt, "prev_row");
+  dtype(save_slot, at::kInt, "save_slot");
+  TORCH_CHECK(q.dim() == 3 && v.dim() == 3 && state.dim() == 4, "delta_rule: q [T, G, N], v [T, H, P], state [slots, H, N, P]");
+  const int64_t T = q.size(0), G = q.size(1), N = q.size(2), H = v.size(1), P = v.size(2);
+  TORCH_CHECK(k.sizes() == q.sizes() && v.size(0) == T && state.size(1) == H && state.size(2) == N && state.size(3) == P &&
+                  out.numel() == T * H * P && A_log.numel() == H && dt_bias.numel() == (channel ? H * N : H) &&
+                  prev_row.numel() >= T && save_slot.numel() >= T, "delta_rule: shapes");
+  TORCH_CHECK(G > 0 && H % G == 0 && H <= 65535 && N >= 1 && N <= 256 && P >= 1 && runs >= 0 && runs <= 65535,
+              "delta_rule: sizes (key channels up to 256)");
+  DeltaRuleArgs a{};
+  a.ldd = view2(dz, 1, T, channel ? H * N : H, "dz");
+  a.ldb = view2(bz, 1, T, H, "bz");
+  if (cu_q.has_value()) {
+    dtype(*cu_q, at::kInt, "cu_q");
+    TORCH_CHECK(cu_q->numel() >= runs + 1, "delta_rule: cu_q too short");
+    a.cu_q = ptr<int>(*cu_q);
+  } else {
+    TORCH_CHECK(runs <= T, "delta_rule: more runs than rows");
+  }
+  if (tiles.has_value()) {
+    TORCH_CHECK(ws.has_value() && cu_q.has_value(), "delta_rule: tiles need ws and cu_q");
+    dtype(*tiles, at::kInt, "tiles");
+    dtype(*ws, at::kFloat, "ws");
+    TORCH_CHECK(tiles->dim() == 2 && tiles->size(1) == 2 && ws->numel() >= T * H * (64 + (channel ? N : 4)),
+                "delta_rule: tiles [n, 2], ws [T, H, 64 + (channel ? N : 4)]");
+    a.tiles = ptr<int>(*tiles);
+    a.ntiles = (int)tiles->size(0);
+    a.ws = ptr<float>(*ws);
+  }
+  a.q = ptr<float>(q);
+  a.k = ptr<float>(k);
+  a.v = v.data_ptr();
+  a.dz = ptr<float>(dz);
+  a.bz = ptr<float>(bz);
+  a.dt_bias = ptr<float>(dt_bias);
+  a.A_log = ptr<float>(A_log);
+  a.state = ptr<float>(state);
+  a.state_stride = state.stride(0);
+  a.prev_row = ptr<int>(prev_row);
+  a.save_slot = ptr<int>(save_slot);
+  a.out = ptr<float>(out);
+  a.T = (int)T, a.H = (int)H, a.G = (int)G, a.N = (int)N, a.P = (int)P, a.hpg = (int)(H / G), a.runs = (int)runs;
+  return launch_delta_rule(a, channel ? 1 : 0, f32, (int)impl, cur_stream(out));
+}
+
 }  // namespace
 
 TORCH_LIBRARY(symmetry_amd_hybrid, m) {
@@ -798,7 +952,8 @@ TORCH_LIBRARY(symmetry_amd_hybrid, m) {
       "float q_scale, int H, int N, int P, int hpg, Tensor(a!) state, Tensor? cu_q, Tensor prev_row, Tensor save_slot, "
       "int runs, Tensor(b!) out, Tensor(c!)? mout) -> ()",
       &decay_scan);
-  m.def("gated_group_norm(Tensor y, Tensor gate, Tensor w, float eps, int group, bool gate_first, Tensor(a!) out) -> ()",
+  m.def("gated_group_norm(Tensor y, Tensor gate, Tensor w, float eps, int group, bool gate_first, Tensor(a!) out, "
+        "bool sigmoid=False) -> ()",
         &gated_group_norm);
   m.def(
       "causal_conv_silu(Tensor xin, Tensor w, Tensor b, Tensor(a!) state, Tensor? cu_q, Tensor? row_seq, Tensor prev_row, "
@@ -855,5 +1010,19 @@ TORCH_LIBRARY(symmetry_amd_hybrid, m) {
       &conv_qkv_cache);
   m.def("memory_norm_gate(Tensor y, Tensor m, Tensor gate, Tensor w, float eps, Tensor(a!) out) -> ()", &memory_norm_gate);
   m.def("clamped_glu(Tensor gu, float limit, float alpha, Tensor(a!) out) -> ()", &hyb_clamped_glu);
+  m.def(
+      "residual_layer_norm(Tensor(a!) x, Tensor? base, Tensor? a, Tensor? b, Tensor? w, Tensor? bias, float eps, Tensor? rows, "
+      "Tensor(b!)? out) -> ()",
+      &residual_layer_norm);
+  m.def(
+      "conv_silu_qkv(Tensor z, Tensor w, Tensor(a!) state, Tensor? cu_q, Tensor? row_seq, Tensor prev_row, Tensor? save_slot, "
+      "int runs, int G, int N, int H, int P, float q_scale, float unit_eps, Tensor(b!) q_out, Tensor(c!) k_out, "
+      "Tensor(d!) v_out) -> ()",
+      &conv_silu_qkv);
+  m.def(
+      "delta_rule(bool channel, Tensor q, Tensor k, Tensor v, Tensor dz, Tensor dt_bias, Tensor A_log, Tensor bz, "
+      "Tensor(a!) state, Tensor? cu_q, Tensor prev_row, Tensor save_slot, int runs, Tensor(b!) out, Tensor? tiles, "
+      "Tensor(c!)? ws, int impl) -> int",
+      &delta_rule);
   m.def("logit_softcap(Tensor(a!) logits, float cap) -> ()", &logit_softcap);
 }

@@ -133,12 +133,15 @@ void layer_norm(const Tensor& x, const OptTensor& rows, const Tensor& w, double 
                     f32, cur_stream(x));
 }
 
-void latent_prep(const Tensor& z, int64_t q_rank, int64_t kv_rank, int64_t rot, const Tensor& wq, const OptTensor& wkv,
-                 double eps, const Tensor& positions, const Tensor& slots, const Tensor& rope, Tensor& cq,
+void latent_prep(const Tensor& z, int64_t q_rank, int64_t kv_rank, int64_t rot, const OptTensor& wq, const OptTensor& wkv,
+                 double eps, const Tensor& positions, const Tensor& slots, const Tensor& rope, const OptTensor& cq,
                  const OptTensor& cache, int64_t half_dims) {
   const int f32 = act(z, "z", false);
-  same_act(wq, f32, "wq");
-  same_act(cq, f32, "cq");
+  TORCH_CHECK(q_rank >= 0 && (q_rank == 0 || (wq.has_value() && cq.has_value())), "latent_prep: the query latent needs wq and cq");
+  if (q_rank > 0) {
+    same_act(*wq, f32, "wq");
+    same_act(*cq, f32, "cq");
+  }
   dtype(positions, at::kInt, "positions");
   dtype(slots, at::kInt, "slots");
   dtype(rope, at::kFloat, "rope");
@@ -153,8 +156,8 @@ void latent_prep(const Tensor& z, int64_t q_rank, int64_t kv_rank, int64_t rot, 
   a.q_rank = (int)q_rank;
   a.kv_rank = (int)kv_rank;
   a.rot = (int)rot;
-  TORCH_CHECK(z.dim() == 2 && wq.numel() == q_rank && cq.numel() == T * q_rank && positions.numel() >= T &&
-                  slots.numel() >= T && rot % 2 == 0, "latent_prep: shapes");
+  TORCH_CHECK(z.dim() == 2 && (q_rank == 0 || (wq->numel() == q_rank && cq->numel() == T * q_rank)) &&
+                  positions.numel() >= T && slots.numel() >= T && rot % 2 == 0, "latent_prep: shapes");
   if (kv_rank > 0) {
     TORCH_CHECK(wkv.has_value() && cache.has_value(), "latent_prep: kv part needs wkv and cache");
     same_act(*wkv, f32, "wkv");
@@ -166,12 +169,12 @@ void latent_prep(const Tensor& z, int64_t q_rank, int64_t kv_rank, int64_t rot, 
   } else {
     TORCH_CHECK(zcols == q_rank, "latent_prep: z width");
   }
-  a.wq = wq.data_ptr();
+  a.wq = q_rank > 0 ? wq->data_ptr() : nullptr;
   a.eps = (float)eps;
   a.positions = ptr<int>(positions);
   a.slots = ptr<int>(slots);
   a.rope = ptr<float>(rope);
-  a.cq = cq.data_ptr();
+  a.cq = q_rank > 0 ? cq->data_ptr() : nullptr;
   launch_latent_prep(a, (int)T, f32, cur_stream(z));
 }
 
@@ -191,7 +194,8 @@ void rope_pairs(const Tensor& src, Tensor& dst, const Tensor& positions, const T
 
 int64_t latent_attn(const Tensor& q, const Tensor& cache, const Tensor& block_tables, const Tensor& row_seq,
                     const Tensor& positions, double scale, int64_t kv_rank, Tensor& out, const OptTensor& part_o,
-                    const OptTensor& part_ml, const OptTensor& tiles, const OptTensor& cu_q, int64_t impl, int64_t window) {
+                    const OptTensor& part_ml, const OptTensor& tiles, const OptTensor& cu_q, int64_t impl, int64_t window,
+                    const OptTensor& sink, const OptTensor& gate) {
   const int f32 = act(q, "q");
   same_act(cache, f32, "cache");
   same_act(out, f32, "out");
@@ -237,6 +241,18 @@ int64_t latent_attn(const Tensor& q, const Tensor& cache, const Tensor& block_ta
   a.positions = ptr<int>(positions);
   a.out = out.data_ptr();
   a.scale = (float)scale;
+  if (sink.has_value()) {
+    dtype(*sink, at::kFloat, "sink");
+    TORCH_CHECK(sink->numel() == a.H, "latent_attn: sink [H]");
+    a.sink = ptr<float>(*sink);
+  }
+  if (gate.has_value()) {
+    same_act(*gate, f32, "gate", false);
+    TORCH_CHECK(gate->dim() == 2 && gate->size(0) == a.T && gate->size(1) == a.H && (a.H == 1 || gate->stride(1) == 1),
+                "latent_attn: gate [T, H] with unit inner stride");
+    a.gate = gate->data_ptr();
+    a.ldg = a.T > 1 ? gate->stride(0) : a.H;
+  }
   if (tiles.has_value()) {
     TORCH_CHECK(cu_q.has_value() && !part_o.has_value(), "latent_attn: tiles need cu_q and take no split-KV partials");
     dtype(*tiles, at::kInt, "tiles");
@@ -337,14 +353,14 @@ TORCH_LIBRARY(symmetry_amd_latent, m) {
       &add_layer_norm);
   m.def("layer_norm(Tensor x, Tensor? rows, Tensor w, float eps, Tensor(a!) out) -> ()", &layer_norm);
   m.def(
-      "latent_prep(Tensor z, int q_rank, int kv_rank, int rot, Tensor wq, Tensor? wkv, float eps, Tensor positions, "
-      "Tensor slots, Tensor rope, Tensor(a!) cq, Tensor(b!)? cache, int half_dims) -> ()",
+      "latent_prep(Tensor z, int q_rank, int kv_rank, int rot, Tensor? wq, Tensor? wkv, float eps, Tensor positions, "
+      "Tensor slots, Tensor rope, Tensor(a!)? cq, Tensor(b!)? cache, int half_dims) -> ()",
       &latent_prep);
   m.def("rope_pairs(Tensor src, Tensor(a!) dst, Tensor positions, Tensor rope, int half_dims) -> ()", &rope_pairs);
   m.def(
       "latent_attn(Tensor q, Tensor cache, Tensor block_tables, Tensor row_seq, Tensor positions, float scale, "
       "int kv_rank, Tensor(a!) out, Tensor(b!)? part_o, Tensor(c!)? part_ml, Tensor? tiles, Tensor? cu_q, int impl, "
-      "int window) -> int",
+      "int window, Tensor? sink=None, Tensor? gate=None) -> int",
       &latent_attn);
   m.def("clamped_glu(Tensor gu, float limit, float alpha, Tensor(a!) out) -> ()", &clamped_glu);
   m.def("sigmoid_topk(Tensor x, Tensor Wr, int k, Tensor(a!) ids, Tensor(b!) w) -> ()", &sigmoid_topk);

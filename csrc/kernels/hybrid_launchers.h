@@ -1,5 +1,5 @@
-// Host-side launch entry points of the kernels in hybrid_rows.hip, stream_rows.hip, window_attention.hip and
-// decay_scan.hip: the
+// Host-side launch entry points of the kernels in hybrid_rows.hip, stream_rows.hip, window_attention.hip, decay_scan.hip
+// and delta_rule.hip: the
 // mechanisms of models that put windowed softmax attention beside linear recurrences with decaying state, use
 // state-space layers with a carried convolution, and add mixer and feed-forward to the stream from one norm.
 //
@@ -45,10 +45,10 @@ struct QkvRopeArgs {
   void* v_cache;
 };
 void launch_qkv_rope_cache(const QkvRopeArgs& a, int T, int f32, hipStream_t s);
-// s = silu(gate); gate_first: out = rms_g(y s) w, else out = rms_g(y) w s; rms over groups of `group` columns,
-// w [wlen] repeating over the columns
+// s = silu(gate) or sigmoid(gate); gate_first: out = rms_g(y s) w, else out = rms_g(y) w s; rms over groups of `group`
+// columns, w [wlen] repeating over the columns
 void launch_gated_group_norm(const float* y, const void* gate, long long ldg, const float* w, int wlen, float eps,
-                             int group, int gate_first, void* out, int T, int C, int f32, hipStream_t s);
+                             int group, int gate_first, int sigmoid, void* out, int T, int C, int f32, hipStream_t s);
 // run i = rows cu_q[i] .. cu_q[i + 1] (cu_q null: row i alone); inputs before a run: state[slot] [taps - 1][C] where
 // prev_row[first] <= -2 (slot = -(v + 2)), else zero.  out = silu(b + sum_j w[c][taps - 1 - j] x[t - j][c])
 struct ConvArgs {
@@ -179,6 +179,31 @@ struct DecayScanArgs {
 };
 void launch_decay_scan(const DecayScanArgs& a, int f32, hipStream_t s);
 
+// ---- delta_rule.hip ------------------------------------------------------------------------------------
+// S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  out = S^T q  per head over every run, beta = sigmoid(bz[h]),
+// log g = -exp(A_log[h]) softplus(dz + dt_bias): one per head, or (channel) one per head and key channel
+struct DeltaRuleArgs {
+  const float* q;       // [T][G][N]
+  const float* k;       // [T][G][N]
+  const void* v;        // [T][H][P] activation dtype
+  const float* dz; long long ldd;   // [T][H], channel: [T][H N]
+  const float* bz; long long ldb;   // [T][H]
+  const float* dt_bias; // [H], channel: [H N]
+  const float* A_log;   // [H]
+  float* state;         // [slots][H][N][P]
+  long long state_stride;
+  const int* cu_q;      // runs (null: every row its own run)
+  const int* prev_row;
+  const int* save_slot;
+  float* out;           // [T][H][P]
+  float* ws;            // chunked form: [T][H][64 + (channel ? N : 4)]
+  const int* tiles;     // chunked form: 64-row tiles (sequence, first row within the run)
+  int ntiles;
+  int T, H, G, N, P, hpg, runs;
+};
+// impl 0: the chunked form where tiles and ws are given; 1: token by token.  Returns the form used.
+int launch_delta_rule(const DeltaRuleArgs& a, int channel, int f32, int impl, hipStream_t s);
+
 // ---- stream_rows.hip -----------------------------------------------------------------------------------
 // x[row][s] (s < S) = table[token] + pair_table[(p mul_prev + token mul_cur) mod buckets]; p = the token of row
 // prev_row[row] (>= 0), tok_state[-(prev_row[row] + 2)] (<= -2) or none (-1: row `buckets` of pair_table); pair_table null:
@@ -236,6 +261,40 @@ void launch_conv_qkv_cache(const ConvQkvArgs& a, int f32, hipStream_t s);
 // y [T][H][P + 1] (column P: n . q), m [T][H]: out = y / (max(|n . q|, exp(-m)) + 1e-6) / rms_head * w * sigmoid(gate)
 void launch_memory_norm_gate(const float* y, const float* m, const void* gate, long long ldg, const float* w, float eps,
                              void* out, int T, int H, int P, int f32, hipStream_t s);
+// x = base + a + b (base null: x; a, b optional; base fp32, a and b bf16 or fp32: *_f32) for the rows < T; with out:
+// out[i] = (x[rows ? rows[i] : i] - mean) / sqrt(var + eps) * w + bias for i < n (rows: without a sum)
+struct ResidualLnArgs {
+  float* x;
+  const float* base;
+  const void* a; int a_f32;
+  const void* b; int b_f32;
+  const float* w;
+  const float* bias;
+  float eps;
+  const long long* rows;
+  void* out;            // [n][d] activation dtype or null
+  int n, d;             // rows of the launch
+};
+void launch_residual_layer_norm(const ResidualLnArgs& a, int f32, hipStream_t s);
+// z[t] = q (G N) | k (G N) | v (H P) through the causal per-channel convolution w [C][taps] (as for ConvQkvArgs), then
+// silu; q and k heads to unit length y / sqrt(sum y^2 + eps), q times q_scale -> q_out, k_out fp32; v -> v_out.  save_slot
+// with cu_q null: the launch moves the row's carried taps on itself
+struct ConvSiluArgs {
+  const void* z; long long ldz;
+  const void* w;        // [C][taps] activation dtype
+  void* state;          // [slots][taps - 1][C] activation dtype
+  long long state_stride;
+  const int* cu_q;
+  const int* row_seq;
+  const int* prev_row;
+  const int* save_slot;
+  float* q_out;         // [T][G][N]
+  float* k_out;         // [T][G][N]
+  void* v_out;          // [T][H][P] activation dtype
+  float q_scale, eps;
+  int T, C, taps, G, N, H, P;
+};
+void launch_conv_silu_qkv(const ConvSiluArgs& a, int f32, hipStream_t s);
 // x = cap tanh(x / cap)
 void launch_logit_softcap(float* x, long long n, float cap, hipStream_t s);
 // glu_moe.hip (declared with the latent family's launchers): launch_clamped_glu, the expert-segment kernels

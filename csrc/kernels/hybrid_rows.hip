@@ -5,7 +5,7 @@
 //   rms_norm_rows       norm of (gathered) stream rows into the activation dtype
 //   residual_mix_norm   x += sa (a + bias) + sb b + sc c in fp32, and the next layer's normalised input from the same pass
 //   qkv_rope_cache      bias + scaled interleaved-pair rotary of q / k, paged key / value cache write
-//   gated_group_norm    silu gate and RMS norm over column groups, in either order
+//   gated_group_norm    silu or sigmoid gate and RMS norm over column groups, in either order
 //   causal_conv_silu    per-channel causal convolution over a run of rows with carried taps, + silu
 //   conv_state_update   the newest taps - 1 inputs of every run into its sequence's state slot
 //   relu_sq, silu_mul   feed-forward activations on column ranges of a fused projection
@@ -134,8 +134,8 @@ __global__ __launch_bounds__(BT) void qkv_rope_cache_kernel(QkvRopeArgs a) {
 template <typename T, int BT>
 __global__ __launch_bounds__(BT) void gated_group_norm_kernel(const float* __restrict__ y, const T* __restrict__ gate,
                                                               long long ldg, const float* __restrict__ w, int wlen,
-                                                              float eps, int group, int gate_first, T* __restrict__ out,
-                                                              int C) {
+                                                              float eps, int group, int gate_first, int sigmoid,
+                                                              T* __restrict__ out, int C) {
   __shared__ float scratch[BT / 64];
   const int row = blockIdx.x, c0 = blockIdx.y * group;
   const float* yr = y + (long long)row * C + c0;
@@ -143,13 +143,13 @@ __global__ __launch_bounds__(BT) void gated_group_norm_kernel(const float* __res
   float sq = 0.f;
   for (int c = threadIdx.x; c < group; c += BT) {
     float v = yr[c];
-    if (gate_first) v *= silu_exact((float)gr[c]);
+    if (gate_first) v *= sigmoid ? sigmoidf((float)gr[c]) : silu_exact((float)gr[c]);
     sq += v * v;
   }
   const float r = 1.f / sqrtf(block_sum<BT>(sq, scratch) / (float)group + eps);
   T* orow = out + (long long)row * C + c0;
   for (int c = threadIdx.x; c < group; c += BT) {
-    const float g = silu_exact((float)gr[c]);
+    const float g = sigmoid ? sigmoidf((float)gr[c]) : silu_exact((float)gr[c]);
     const float wv = w[(c0 + c) % wlen];
     orow[c] = (T)(gate_first ? yr[c] * g * r * wv : yr[c] * r * wv * g);
   }
@@ -605,9 +605,10 @@ __global__ __launch_bounds__(NT) void gelu_tanh_mul_kernel(const T* __restrict__
 
 // bf16, F and both row strides multiples of 8, 16-byte aligned views: eight columns per thread (prompt-sized launches
 // are bandwidth-bound)
-__global__ __launch_bounds__(NT) void gelu_tanh_mul_vec_kernel(const bf16* __restrict__ g, long long ldg,
-                                                               const bf16* __restrict__ u, long long ldu,
-                                                               bf16* __restrict__ out, long long nvec, int F) {
+template <bool GELU>
+__global__ __launch_bounds__(NT) void glu_vec_kernel(const bf16* __restrict__ g, long long ldg,
+                                                     const bf16* __restrict__ u, long long ldu,
+                                                     bf16* __restrict__ out, long long nvec, int F) {
   const long long i = (long long)blockIdx.x * NT + threadIdx.x;
   if (i >= nvec) return;
   const int fv = F >> 3;
@@ -617,7 +618,7 @@ __global__ __launch_bounds__(NT) void gelu_tanh_mul_vec_kernel(const bf16* __res
   load8(g + r * ldg + c, gv);
   load8(u + r * ldu + c, uv);
 #pragma unroll
-  for (int j = 0; j < 8; ++j) y[j] = gelu_tanh_exact(gv[j]) * uv[j];
+  for (int j = 0; j < 8; ++j) y[j] = (GELU ? gelu_tanh_exact(gv[j]) : silu_exact(gv[j])) * uv[j];
   store8(out + r * F + c, y);
 }
 
@@ -689,18 +690,18 @@ void launch_qkv_rope_cache(const QkvRopeArgs& a, int T_, int f32, hipStream_t s)
 }
 
 void launch_gated_group_norm(const float* y, const void* gate, long long ldg, const float* w, int wlen, float eps,
-                             int group, int gate_first, void* out, int T_, int C, int f32, hipStream_t s) {
+                             int group, int gate_first, int sigmoid, void* out, int T_, int C, int f32, hipStream_t s) {
   if (T_ <= 0) return;
   dim3 grid(T_, C / group);
   if (group <= 256) {
     DISPATCH_T(f32, (gated_group_norm_kernel<T, 64><<<grid, 64, 0, s>>>(y, (const T*)gate, ldg, w, wlen, eps, group,
-                                                                          gate_first, (T*)out, C));)
+                                                                          gate_first, sigmoid, (T*)out, C));)
   } else if (wide_rows(T_, group)) {
     DISPATCH_T(f32, (gated_group_norm_kernel<T, 1024><<<grid, 1024, 0, s>>>(y, (const T*)gate, ldg, w, wlen, eps, group,
-                                                                              gate_first, (T*)out, C));)
+                                                                              gate_first, sigmoid, (T*)out, C));)
   } else {
     DISPATCH_T(f32, (gated_group_norm_kernel<T, NT><<<grid, NT, 0, s>>>(y, (const T*)gate, ldg, w, wlen, eps, group,
-                                                                          gate_first, (T*)out, C));)
+                                                                          gate_first, sigmoid, (T*)out, C));)
   }
 }
 
@@ -721,9 +722,20 @@ void launch_relu_sq(const void* a, long long lda, void* out, int R, int F, int f
   DISPATCH_T(f32, relu_sq_kernel<T><<<ew_grid((long long)R * F), NT, 0, s>>>((const T*)a, lda, (T*)out, R, F);)
 }
 
+// eight columns per thread where the views allow it
+template <bool GELU>
+bool glu_vec(const void* gate, long long ldg, const void* up, long long ldu, void* out, int R, int F, int f32, hipStream_t s) {
+  const auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  if (f32 || F % 8 || ldg % 8 || ldu % 8 || !al(gate) || !al(up) || !al(out)) return false;
+  const long long nvec = (long long)R * F / 8;
+  glu_vec_kernel<GELU><<<(unsigned)((nvec + NT - 1) / NT), NT, 0, s>>>((const bf16*)gate, ldg, (const bf16*)up, ldu,
+                                                                       (bf16*)out, nvec, F);
+  return true;
+}
+
 void launch_silu_mul(const void* gate, long long ldg, const void* up, long long ldu, void* out, int R, int F, int f32,
                      hipStream_t s) {
-  if (R <= 0) return;
+  if (R <= 0 || glu_vec<false>(gate, ldg, up, ldu, out, R, F, f32, s)) return;
   DISPATCH_T(f32, silu_mul_kernel<T><<<ew_grid((long long)R * F), NT, 0, s>>>((const T*)gate, ldg, (const T*)up, ldu,
                                                                               (T*)out, R, F);)
 }
@@ -813,14 +825,7 @@ void launch_qk_norm_cache(const QkNormArgs& a, int T_, int f32, hipStream_t s) {
 
 void launch_gelu_tanh_mul(const void* gate, long long ldg, const void* up, long long ldu, void* out, int R, int F, int f32,
                           hipStream_t s) {
-  if (R <= 0) return;
-  const auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
-  if (!f32 && F % 8 == 0 && ldg % 8 == 0 && ldu % 8 == 0 && al(gate) && al(up) && al(out)) {
-    const long long nvec = (long long)R * F / 8;
-    gelu_tanh_mul_vec_kernel<<<(unsigned)((nvec + NT - 1) / NT), NT, 0, s>>>((const bf16*)gate, ldg, (const bf16*)up, ldu,
-                                                                           (bf16*)out, nvec, F);
-    return;
-  }
+  if (R <= 0 || glu_vec<true>(gate, ldg, up, ldu, out, R, F, f32, s)) return;
   DISPATCH_T(f32, gelu_tanh_mul_kernel<T><<<ew_grid((long long)R * F), NT, 0, s>>>((const T*)gate, ldg, (const T*)up,
                                                                                    ldu, (T*)out, R, F);)
 }

@@ -15,7 +15,8 @@
 //   rope_pairs    rotary of a strided [T][H][rot] slice: interleaved pairs (dimension 2i with 2i + 1) or the half
 //                 layout (dimension i with i + dims / 2, dimensions past dims passing)
 //   latent_attn   causal softmax attention over the paged latent cache, optionally limited to a sliding window of
-//                 the newest keys; scores, weights and accumulators fp32.
+//                 the newest keys, with a per-head sink in the denominator and a per-head sigmoid gate on the output;
+//                 scores, weights and accumulators fp32.
 //                 Two implementations: the MFMA kernel (bf16, tiled shapes) and a one-wave-per-(row, head) kernel
 //                 for every other shape and for the 32-bit model.
 //
@@ -49,20 +50,38 @@ SYM_DEV void pair_entries(int p, int half_dims, int& e0, int& e1) {
   }
 }
 
+// The last step of a (row, head)'s softmax: the factor on its accumulated sum.  m, l: running maximum and sum of the
+// weights e^(score - m); a sink is one more logit in the denominator, so the factor is 1 / (l + e^(sink - m)) in a form
+// that overflows for no sink; times the sigmoid of the head's gate.
+template <typename T>
+SYM_DEV float out_factor(const LatentAttnArgs& a, long long row, int h, float m, float l) {
+  float f = 1.f;
+  if (a.sink) {
+    const float sk = a.sink[h], M = fmaxf(m, sk);
+    f = expf(m - M);
+    l = l * f + expf(sk - M);
+  }
+  f /= l;
+  if (a.gate) f /= 1.f + expf(-(float)reinterpret_cast<const T*>(a.gate)[row * a.ldg + h]);
+  return f;
+}
+
 template <typename T>
 __global__ __launch_bounds__(NT) void latent_prep_kernel(LatentPrepArgs a) {
   __shared__ float scratch[NT / 64];
   const int row = blockIdx.x;
   const T* z = (const T*)a.z + (long long)row * a.nz;
   float ss = 0.f;
-  for (int c = threadIdx.x; c < a.q_rank; c += NT) {
-    const float v = (float)z[c];
-    ss += v * v;
+  if (a.q_rank > 0) {   // (launch-uniform)
+    for (int c = threadIdx.x; c < a.q_rank; c += NT) {
+      const float v = (float)z[c];
+      ss += v * v;
+    }
+    const float rq = 1.f / sqrtf(block_sum<NT>(ss, scratch) / (float)a.q_rank + a.eps);
+    T* cq = (T*)a.cq + (long long)row * a.q_rank;
+    const T* wq = (const T*)a.wq;
+    for (int c = threadIdx.x; c < a.q_rank; c += NT) cq[c] = (T)((float)z[c] * rq * (float)wq[c]);
   }
-  const float rq = 1.f / sqrtf(block_sum<NT>(ss, scratch) / (float)a.q_rank + a.eps);
-  T* cq = (T*)a.cq + (long long)row * a.q_rank;
-  const T* wq = (const T*)a.wq;
-  for (int c = threadIdx.x; c < a.q_rank; c += NT) cq[c] = (T)((float)z[c] * rq * (float)wq[c]);
   if (a.kv_rank == 0) return;
   const int slot = a.slots[row];
   const T* zk = z + a.q_rank;
@@ -191,7 +210,7 @@ __global__ __launch_bounds__(64) void latent_attn_wave_kernel(LatentAttnArgs a) 
   }
   if (a.parts == 1) {
     T* out = (T*)a.out + ((long long)row * a.H + h) * a.kv_rank;
-    const float inv = 1.f / l;
+    const float inv = out_factor<T>(a, row, h, m, l);
 #pragma unroll
     for (int i = 0; i < MAXR; ++i) {
       const int c = lane + 64 * i;
@@ -240,7 +259,7 @@ __global__ __launch_bounds__(256) void latent_attn_merge_kernel(LatentAttnArgs a
   l = wave_sum(l);
   if (lane == 0) stat[4 + wave] = l;
   __syncthreads();
-  const float inv = 1.f / (stat[4] + stat[5] + stat[6] + stat[7]);
+  const float inv = out_factor<T>(a, row, h, m, stat[4] + stat[5] + stat[6] + stat[7]);
   float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
   for (int p = wave; p < np; p += 4) {
@@ -492,7 +511,7 @@ __global__ __launch_bounds__(64 * NW) void latent_attn_mfma_kernel(LatentAttnArg
   // o[dt][i]: dim (dh * rtd + dt) * 16 + g * 4 + i of query vector n
   if (a.parts == 1) {
     bf16* out = (bf16*)a.out + ((long long)qrow * H + head) * r + dh * rtd * 16;
-    const float inv = 1.f / l;
+    const float inv = out_factor<bf16>(a, qrow, head, m, l);
 #pragma unroll
     for (int dt = 0; dt < RTD; ++dt)
       if (EXACT || dt < rtd) {

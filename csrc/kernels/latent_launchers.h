@@ -28,7 +28,8 @@ void launch_layer_norm(const float* x, const long long* rows, const void* w, flo
 // ---- latent_attention.hip ----------------------------------------------------------------------------
 struct LatentPrepArgs {
   const void* z;        // [T][nz] projections of the mixer input: q latent | kv latent | shared rotary key
-  int nz, q_rank, kv_rank, rot;  // nz: row stride of z; kv_rank == 0: no kv part (the layer attends another's cache)
+  int nz, q_rank, kv_rank, rot;  // nz: row stride of z; q_rank == 0: no query latent; kv_rank == 0: no kv part (the layer
+                                 // attends another's cache)
   int half_dims;        // 0: rotary pairs (2i, 2i + 1); > 0: entry i pairs with i + half_dims / 2, later entries pass
   const void* wq;       // [q_rank] norm weight
   const void* wkv;      // [kv_rank]
@@ -59,6 +60,9 @@ struct LatentAttnArgs {
   int parts, part_tokens;  // split-KV: partition p of a row covers part_tokens keys from first + p * part_tokens on,
                            // first = the row's first visible key
   float scale;
+  const float* sink;       // [H] or null: the softmax's denominator also holds exp(sink[h])
+  const void* gate;        // [T][H] (row stride ldg) or null: output times sigmoid(gate)
+  long long ldg;
   // prompt form of the MFMA kernel: 64-row query tiles (sequence, first row within the sequence's run) over the
   // runs cu_q[seq] .. cu_q[seq + 1]; nullptr: one query row per sequence (decode steps)
   const int* tiles;

@@ -9,6 +9,10 @@
 //                        (a workgroup per (row, head))
 //   memory_norm_gate     o / (max(|n . q|, exp(-m)) + 1e-6), unit RMS per head, weight, sigmoid gate
 //   logit_softcap        cap tanh(logits / cap)
+//   residual_layer_norm  x = base + a + b on the fp32 stream and the next sublayer's layer norm (weight, bias) from the same
+//                        pass; also the gathered norm in front of the output head
+//   conv_silu_qkv        causal per-channel convolution of q | k | v with carried taps, silu, unit-vector q / k heads (a wave
+//                        per (rows, head))
 //
 // One workgroup per row unless noted; columns strided over the threads (coalesced), any width.  All statistics, mixing
 // and sums are fp32; only the stored activations take the activation dtype T (bf16 or float).
@@ -237,6 +241,183 @@ __global__ __launch_bounds__(64) void memory_norm_gate_kernel(const float* __res
     orow[c] = (T)(yr[c] / den * r * w[(long long)h * P + c] * sigmoidf((float)gr[c]));
 }
 
+// Four columns of a row, fp32 or bf16
+SYM_DEV float4 ld4(const void* p, int f32, long long i) {
+  if (f32) return *reinterpret_cast<const float4*>(reinterpret_cast<const float*>(p) + i);
+  const bf16x4 v = *reinterpret_cast<const bf16x4*>(reinterpret_cast<const bf16*>(p) + i);
+  return make_float4((float)v[0], (float)v[1], (float)v[2], (float)v[3]);
+}
+SYM_DEV void st4(float* p, const float4& v) { *reinterpret_cast<float4*>(p) = v; }
+SYM_DEV void st4(bf16* p, const float4& v) {
+  bf16x4 o;
+  o[0] = (bf16)v.x, o[1] = (bf16)v.y, o[2] = (bf16)v.z, o[3] = (bf16)v.w;
+  *reinterpret_cast<bf16x4*>(p) = o;
+}
+
+// One workgroup per row; VPT > 0: the row in registers, VPT vectors of four columns per thread (d % 4 == 0, d <= 4 BT VPT);
+// VPT == 0: any width, columns strided over the threads and re-read (each thread those it wrote itself)
+template <typename T, int BT, int VPT>
+__global__ __launch_bounds__(BT) void residual_layer_norm_kernel(ResidualLnArgs a) {
+  __shared__ float scratch[BT / 64];
+  const int row = blockIdx.x, d = a.d;
+  const long long xrow = a.rows ? a.rows[row] : (long long)row;
+  const long long o = (long long)row * d;
+  float* x = a.x + xrow * d;
+  const float* base = a.base ? a.base + xrow * d : x;
+  const bool upd = a.base || a.a || a.b;
+  float sum = 0.f, sq = 0.f;
+  if constexpr (VPT > 0) {
+    float4 v[VPT];
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int c = 4 * (threadIdx.x + BT * i);
+      v[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (c < d) {
+        v[i] = *reinterpret_cast<const float4*>(base + c);
+        if (a.a) {
+          const float4 t = ld4(a.a, a.a_f32, o + c);
+          v[i].x += t.x, v[i].y += t.y, v[i].z += t.z, v[i].w += t.w;
+        }
+        if (a.b) {
+          const float4 t = ld4(a.b, a.b_f32, o + c);
+          v[i].x += t.x, v[i].y += t.y, v[i].z += t.z, v[i].w += t.w;
+        }
+        if (upd) st4(x + c, v[i]);
+        sum += (v[i].x + v[i].y) + (v[i].z + v[i].w);
+      }
+    }
+    if (!a.out) return;     // (launch-uniform)
+    float4 w[VPT], bs[VPT];   // (loads under the reductions)
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int c = 4 * (threadIdx.x + BT * i);
+      if (c < d) {
+        w[i] = *reinterpret_cast<const float4*>(a.w + c);
+        bs[i] = *reinterpret_cast<const float4*>(a.bias + c);
+      }
+    }
+    const float mean = block_sum<BT>(sum, scratch) / (float)d;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      if (4 * (int)(threadIdx.x + BT * i) < d) {
+        v[i].x -= mean, v[i].y -= mean, v[i].z -= mean, v[i].w -= mean;
+        sq += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+      }
+    }
+    const float r = 1.f / sqrtf(block_sum<BT>(sq, scratch) / (float)d + a.eps);
+    T* out = reinterpret_cast<T*>(a.out) + o;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int c = 4 * (threadIdx.x + BT * i);
+      if (c < d)
+        st4(out + c, make_float4(v[i].x * r * w[i].x + bs[i].x, v[i].y * r * w[i].y + bs[i].y, v[i].z * r * w[i].z + bs[i].z,
+                                 v[i].w * r * w[i].w + bs[i].w));
+    }
+  } else {
+    for (int c = threadIdx.x; c < d; c += BT) {
+      float v = base[c];
+      if (a.a) v += ldf(a.a, a.a_f32, o + c);
+      if (a.b) v += ldf(a.b, a.b_f32, o + c);
+      if (upd) x[c] = v;
+      sum += v;
+    }
+    if (!a.out) return;
+    const float mean = block_sum<BT>(sum, scratch) / (float)d;
+    for (int c = threadIdx.x; c < d; c += BT) sq += (x[c] - mean) * (x[c] - mean);
+    const float r = 1.f / sqrtf(block_sum<BT>(sq, scratch) / (float)d + a.eps);
+    T* out = reinterpret_cast<T*>(a.out) + o;
+    for (int c = threadIdx.x; c < d; c += BT) out[c] = (T)((x[c] - mean) * r * a.w[c] + a.bias[c]);
+  }
+}
+
+// A wave per (ROWS consecutive rows, head of q | k | v); a lane owns VC neighbouring channels of the head, PER times over
+// (64 VC PER >= the widest head).  VC = 4: eight- or sixteen-byte accesses (row strides, head sizes and bases permitting).
+template <typename T, int VC, int PER, int ROWS>
+__global__ void conv_silu_qkv_kernel(ConvSiluArgs a) {
+  const int lane = threadIdx.x & 63;
+  const int unit = blockIdx.y * (blockDim.x >> 6) + (threadIdx.x >> 6);
+  if (unit >= 2 * a.G + a.H) return;
+  const int taps = a.taps, C = a.C, keep = taps - 1;
+  const int nq = a.G * a.N;
+  const int kind = unit < a.G ? 0 : (unit < 2 * a.G ? 1 : 2);     // q, k or v head
+  const int hd = unit - kind * a.G;
+  const int width = kind == 2 ? a.P : a.N;
+  const int c0 = kind * nq + hd * width;
+  const T* z = reinterpret_cast<const T*>(a.z);
+  const T* w = reinterpret_cast<const T*>(a.w);
+  for (int row = blockIdx.x * ROWS; row < min(a.T, (int)(blockIdx.x + 1) * ROWS); ++row) {
+    const int s0 = a.cu_q ? a.cu_q[a.row_seq[row]] : row;
+    const int j = row - s0;
+    const int pr = j < keep ? a.prev_row[s0] : -1;
+    const T* st = pr <= -2 ? reinterpret_cast<const T*>(a.state) + (long long)(-(pr + 2)) * a.state_stride : nullptr;
+    const int sv = (!a.cu_q && a.save_slot) ? a.save_slot[row] : -1;
+    T* dst = sv >= 0 && keep ? reinterpret_cast<T*>(a.state) + (long long)sv * a.state_stride : nullptr;
+    float y[PER][VC];
+    float sq = 0.f;
+#pragma unroll
+    for (int u = 0; u < PER; ++u) {
+      const int e = VC * (lane + 64 * u);
+#pragma unroll
+      for (int i = 0; i < VC; ++i) y[u][i] = 0.f;
+      if (e < width) {
+        const int c = c0 + e;
+        T hist[MAX_TAPS][VC];     // hist[b]: the input b places back (b = 0: this row's)
+#pragma unroll
+        for (int b = 0; b < MAX_TAPS; ++b) {
+          if (b < taps) {
+            const T* src = b <= j ? z + (long long)(row - b) * a.ldz + c : (st ? st + (long long)(keep - (b - j)) * C + c : nullptr);
+            if (src) {
+              if constexpr (VC == 4) __builtin_memcpy(hist[b], __builtin_assume_aligned(src, 4 * sizeof(T)), 4 * sizeof(T));
+              else hist[b][0] = src[0];
+            } else {
+#pragma unroll
+              for (int i = 0; i < VC; ++i) hist[b][i] = (T)0.f;
+            }
+          }
+        }
+#pragma unroll
+        for (int b = 0; b < MAX_TAPS; ++b)
+          if (b < taps)
+#pragma unroll
+            for (int i = 0; i < VC; ++i) y[u][i] += (float)w[(long long)(c + i) * taps + keep - b] * (float)hist[b][i];
+#pragma unroll
+        for (int i = 0; i < VC; ++i) {
+          y[u][i] *= sigmoidf(y[u][i]);
+          sq += y[u][i] * y[u][i];
+        }
+        // rows that are runs of their own: this lane alone reads and writes its channels of the row's slot, so the carried
+        // taps move on here (place m holds the input keep - m back from the next token)
+        if (dst) {
+#pragma unroll
+          for (int b = 0; b < MAX_TAPS - 1; ++b)
+            if (b < keep) {
+              T* o = dst + (long long)(keep - 1 - b) * C + c;
+              if constexpr (VC == 4) __builtin_memcpy(__builtin_assume_aligned(o, 4 * sizeof(T)), hist[b], 4 * sizeof(T));
+              else o[0] = hist[b][0];
+            }
+        }
+      }
+    }
+    float r = 1.f;
+    if (kind < 2) r = 1.f / sqrtf(wave_sum(sq) + a.eps) * (kind == 0 ? a.q_scale : 1.f);
+#pragma unroll
+    for (int u = 0; u < PER; ++u) {
+      const int e = VC * (lane + 64 * u);
+      if (e < width) {
+        if (kind < 2) {
+          float* o = (kind == 0 ? a.q_out : a.k_out) + (long long)row * nq + hd * width + e;
+          if constexpr (VC == 4) st4(o, make_float4(y[u][0] * r, y[u][1] * r, y[u][2] * r, y[u][3] * r));
+          else o[0] = y[u][0] * r;
+        } else {
+          T* o = reinterpret_cast<T*>(a.v_out) + ((long long)row * a.H + hd) * width + e;
+          if constexpr (VC == 4) st4(o, make_float4(y[u][0], y[u][1], y[u][2], y[u][3]));
+          else o[0] = (T)y[u][0];
+        }
+      }
+    }
+  }
+}
+
 __global__ __launch_bounds__(NT) void logit_softcap_kernel(float* __restrict__ x, long long n, float cap) {
   for (long long i = (long long)blockIdx.x * NT + threadIdx.x; i < n; i += (long long)gridDim.x * NT)
     x[i] = cap * tanhf(x[i] / cap);
@@ -299,4 +480,47 @@ void launch_logit_softcap(float* x, long long n, float cap, hipStream_t s) {
   if (n <= 0) return;
   const long long blocks = (n + NT - 1) / NT;
   logit_softcap_kernel<<<(unsigned)(blocks < 4096 ? blocks : 4096), NT, 0, s>>>(x, n, cap);
+}
+
+void launch_residual_layer_norm(const ResidualLnArgs& a, int f32, hipStream_t s) {
+  if (a.n <= 0) return;
+  const auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const bool vec = a.d % 4 == 0 && al(a.x) && al(a.base) && al(a.a) && al(a.b) && al(a.w) && al(a.bias) && al(a.out);
+#define LN(BT, VPT) DISPATCH_T(f32, (residual_layer_norm_kernel<T, BT, VPT><<<a.n, BT, 0, s>>>(a));)
+  const int q = a.d / 4;
+  if (!vec || q > 8 * 256) {
+    if (wide_rows(a.n, a.d)) { LN(1024, 0) } else { LN(256, 0) }
+  } else if (q <= 256) {
+    LN(256, 1)
+  } else if (a.n <= 256) {      // a decode-sized launch: more threads per row
+    if (q <= 512) { LN(512, 1) } else if (q <= 1024) { LN(1024, 1) } else { LN(1024, 2) }
+  } else if (q <= 512) {
+    LN(256, 2)
+  } else if (q <= 1024) {
+    LN(256, 4)
+  } else {
+    LN(256, 8)
+  }
+#undef LN
+}
+
+template <int VC, int PER>
+static void conv_silu_rows(const ConvSiluArgs& a, int f32, hipStream_t s) {
+  const int units = 2 * a.G + a.H;
+  if (a.T <= 256) {
+    DISPATCH_T(f32, (conv_silu_qkv_kernel<T, VC, PER, 1><<<dim3(a.T, units), 64, 0, s>>>(a));)
+  } else {
+    DISPATCH_T(f32, (conv_silu_qkv_kernel<T, VC, PER, 4><<<dim3((a.T + 3) / 4, (units + 3) / 4), 256, 0, s>>>(a));)
+  }
+}
+
+void launch_conv_silu_qkv(const ConvSiluArgs& a, int f32, hipStream_t s) {
+  if (a.T <= 0) return;
+  const auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const int wide = a.N > a.P ? a.N : a.P;
+  const bool vec = a.N % 4 == 0 && a.P % 4 == 0 && a.ldz % 4 == 0 && al(a.z) && al(a.state) && a.state_stride % 4 == 0 &&
+                   al(a.q_out) && al(a.k_out) && al(a.v_out);
+  if (vec && wide <= 256) conv_silu_rows<4, 1>(a, f32, s);
+  else if (vec) conv_silu_rows<4, 2>(a, f32, s);      // heads up to 512 wide (checked by the op layer)
+  else conv_silu_rows<1, 8>(a, f32, s);
 }

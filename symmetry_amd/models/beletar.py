@@ -204,7 +204,7 @@ class BeletarLM:
         y = self._buf("del.y", (T, H * V), f32)
         tiles = ws = None
         if prefill and self.dtype == torch.bfloat16 and self.device.type != "cpu":   # (the 32-bit model walks token by token)
-            tiles, ws = b.tiles, self._buf("del.ws", (T, H, 2, ops.DELTA_CHUNK), f32)
+            tiles, ws = b.tiles, self._buf("del.ws", (T, H, ops.delta_ws_cols(m.channel, N)), f32)
         ops.delta_rule(m.channel, q, k, v, dz, P["dt_bias"], P["A_log"], gates[:, :H], cache.rec[n], cu, b.prev_row,
                        b.save_slot, runs, y, tiles, ws)
         gate = self._linear("del.g", self._cols(z, P, "g1"), P["g2"]) if m.channel else self._cols(z, P, "g")

@@ -1055,6 +1055,13 @@ def conv_silu_qkv(z, w, state, cu_q, row_seq, prev_row, runs, G, N, H, P, q_scal
 
 
 DELTA_CHUNK = 32            # tokens per chunk of delta_rule's chunked form (csrc/kernels/delta_rule.hip)
+
+
+def delta_ws_cols(channel: bool, N: int) -> int:
+    """fp32 scratch per (row, head) of delta_rule's chunked form: two rows of C-token matrices and the decays' running sum."""
+    return 2 * DELTA_CHUNK + (N if channel else 4)
+
+
 DELTA_IMPL = 1 if os.environ.get("SYMMETRY_DELTA_RULE", "auto") == "serial" else 0  # A/B: the token-by-token kernel
 
 
@@ -1066,7 +1073,7 @@ def delta_rule(channel, q, k, v, dz, dt_bias, A_log, bz, state, cu_q, prev_row, 
     ``channel`` one per head and key channel (dz fp32 [T, H N]).  q, k fp32 [T, G, N]: head h reads h // (H / G); v [T, H, P]
     bf16 or fp32.  A run starts from state[slot] if prev_row[first] <= -2 (slot = -(v + 2)), else from zero; it ends in
     state[save_slot[last]] (>= 0).  out fp32 [T, H, P].
-    ``tiles`` [n, 2] (sequence, first row of a 64-row tile within the run) + ``ws`` (fp32 scratch of delta_ws_elems):
+    ``tiles`` [n, 2] (sequence, first row of a 64-row tile within the run) + ``ws`` (fp32 scratch [T, H, delta_ws_cols]):
     prompt steps take the chunked form (N <= 256), else and with ``impl=1`` the token-by-token kernel.  Returns the
     implementation used (0 chunked, 1 token by token)."""
     if _gpu(out):

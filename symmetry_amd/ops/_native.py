@@ -85,8 +85,8 @@ _hybrid_loaded = False
 
 
 def hybrid_ops():
-    """``torch.ops.symmetry_amd_hybrid`` (loaded once; built first if the library is missing: five translation units,
-    under a minute).  Raises if it cannot be built or loaded: no eager fallback on the device."""
+    """``torch.ops.symmetry_amd_hybrid`` (loaded once; built first if the library is missing: seven translation units,
+    about a minute).  Raises if it cannot be built or loaded: no eager fallback on the device."""
     global _hybrid_loaded
     with _lock:
         if not _hybrid_loaded:
