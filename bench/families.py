@@ -1,6 +1,6 @@
 #!/usr/bin/env python3
-"""Prefill and decode throughput of a Bozevik, Lemunex, Komazen or Dalalix stack beside the closest Llama / Mixtral stack
-of equal size.
+"""Prefill and decode throughput of a Bozevik, Lemunex, Komazen, Dalalix or Beletar stack beside the closest Llama /
+Mixtral stack of equal size.
 
 Random weights, layer shapes of real models, a few layers each (throughput per layer is what is compared; the
 vocabulary projection is the same size on both sides).  Per size and family, through the engine's own scheduler:
@@ -110,6 +110,29 @@ def _dalalix_pairs():
     }
 
 
+def _beletar_pairs():
+    """Beletar stacks (delta rule with head decays, with channel decays, with head decays, then latent attention) beside the
+    Llama stack of the same width, layer count and feed-forward width, and beside the Lemunex stack (the closest model with
+    matrix-state recurrences) and the Bozevik stack (the closest one with latent attention)."""
+    from symmetry_amd.models.config import ModelConfig, _bozevik_stack, beletar_stack, lemunex_stack
+
+    kw = dict(max_position=8192, bos_token_id=32000, eos_token_ids=(32001, 32002))
+    yarn = (4.0, 4096.0, 32.0, 1.0)
+    small = beletar_stack("beletar-w2048", 32768, 2048, "DCDL", heads=8, kv_heads=8, dim=128, vdim=256, ff=8192, att_heads=16,
+                          embed_scale=8.0, scaling=yarn, **kw)
+    return {
+        "w2048": (small, ModelConfig("llama-w2048", 32768, 2048, 8192, 4, 16, 4, **kw)),
+        "w4096": (beletar_stack("beletar-w4096", 32768, 4096, "DCDL", heads=16, kv_heads=16, dim=128, vdim=256, ff=14336,
+                                att_heads=32, embed_scale=8.0, scaling=yarn, **kw),
+                  ModelConfig("llama-w4096", 32768, 4096, 14336, 4, 32, 8, **kw)),
+        "w2048-lemunex": (small, lemunex_stack("lemunex-w2048", 32768, 2048, "pmmp", heads=16, kv_heads=4, dim=128,
+                                               window=1024, gla_heads=8, gla_dim=128, gla_vdim=256, ssm_heads=64, ssm_vdim=64,
+                                               ssm_state=128, ff=8192, **kw)),
+        "w2048-bozevik": (small, _bozevik_stack("bozevik-w2048", 32768, 2048, 4, heads=16, ff=8192, share_every=0, dim=128,
+                                                rot_dim=64, vdim=128, kv_rank=512, q_rank=1536, **kw)),
+    }
+
+
 def measure(mcfg, prompts: int, plen: int, steps: int, reps: int = 3) -> dict:
     import torch
 
@@ -157,18 +180,19 @@ def measure(mcfg, prompts: int, plen: int, steps: int, reps: int = 3) -> dict:
 
 def main(argv=None) -> int:
     ap = argparse.ArgumentParser(description=__doc__, formatter_class=argparse.RawDescriptionHelpFormatter)
-    ap.add_argument("--sizes", default="w2048,w4096,moe-w2048")
+    ap.add_argument("--sizes", default="w2048,w4096,moe-w2048,w2048-lemunex,w2048-bozevik")
     ap.add_argument("--prompts", type=int, default=8)
     ap.add_argument("--prompt-len", type=int, default=1024)
     ap.add_argument("--decode-steps", type=int, default=64)
-    ap.add_argument("--only", default="", help="bozevik | lemunex | komazen | dalalix | baseline: one side only (profiling)")
-    ap.add_argument("--design", default="bozevik", choices=("bozevik", "lemunex", "komazen", "dalalix"),
+    ap.add_argument("--only", default="", help="bozevik | lemunex | komazen | dalalix | beletar | baseline: one side only (profiling)")
+    ap.add_argument("--design", default="bozevik", choices=("bozevik", "lemunex", "komazen", "dalalix", "beletar"),
                     help="the family measured")
     a = ap.parse_args(argv)
-    pairs = {"bozevik": _pairs, "lemunex": _lemunex_pairs, "komazen": _komazen_pairs, "dalalix": _dalalix_pairs}[a.design]()
+    pairs = {"bozevik": _pairs, "lemunex": _lemunex_pairs, "komazen": _komazen_pairs, "dalalix": _dalalix_pairs,
+             "beletar": _beletar_pairs}[a.design]()
     ratios = {}
     for size in a.sizes.split(","):
-        if size not in pairs:     # (a design without routed layers has no routed size)
+        if size not in pairs:     # (not every design has every size)
             continue
         boz, base = pairs[size]
         rows = {}

@@ -21,14 +21,18 @@
 //        u_i = beta_i (v_i - (k_i e^(G_i))^T S_0 - sum_{j < i} Akk_ij u_j),      Akk_ij = sum_n k_i k_j e^(G_i - G_j)
 //        o_i = (q_i e^(G_i))^T S_0 + sum_{j <= i} Aqk_ij u_j                      (every exponent <= 0: nothing overflows)
 //        S_C = e^(G_C) S_0 + sum_j (k_j e^(G_C - G_j)) u_j^T
-//    delta_chunk_prep_kernel (one workgroup per chunk and head, all chunks at once) evaluates Akk, Aqk -- the exponents of
-//    differences taken per (i, j, channel), so strong decays are exact -- and T = (I + diag(beta) Akk)^-1 diag(beta) by
-//    forward substitution.  delta_chunk_scan_kernel (grid (P / 64, heads, runs)) then walks a run's chunks with
+//    delta_chunk_prep_kernel (one workgroup per chunk and head, all chunks at once) evaluates Akk, Aqk and T = (I +
+//    diag(beta) Akk)^-1 diag(beta) by forward substitution.  One decay per head: the scores are matrix products, times
+//    e^(G_i - G_j).  Decays per channel: inside the two diagonal 16 x 16 tiles the exponents of differences are taken per
+//    (i, j, channel) on the vector unit; the tile below them factors at the end of the first half, e^(G_i - G_15) e^(G_15 -
+//    G_j), both exponents <= 0, and is a matrix product again.
+//    delta_chunk_scan_kernel (grid (P / 64, heads, runs)) then walks a run's chunks with
 //        R = V - Kt S,   U = T R,   O = Qt S + Aqk U,   S <- D S + Kh^T U
 //    as fp32 matrix products (v_mfma_f32_16x16x4_f32).  A wave owns 16 value columns and ALL of N: its state stays in
 //    accumulator registers for the whole run, and since an accumulator's rows are 4 (lane / 16) + r and a B operand's
 //    contraction index is lane / 16, register r of the state IS the B operand of a step that contracts over the rows
 //    4 g + r (the A operand is read in the same order: one 16-byte LDS read feeds four steps).  The same holds for R and U.
+//    Four waves multiply, four others stage the next chunk (loads, exponentials, LDS) on the same SIMDs meanwhile.
 #include "common.h"
 #include "hybrid_launchers.h"
 
@@ -193,11 +197,23 @@ constexpr int LC = C + 4;        // LDS pitch of a [.][C] matrix
 // scratch per (row, head): row of T [C] | row of Aqk [C] | G: N key channels, or one value in four
 SYM_DEV int ws_cols(bool channel, int N) { return 2 * C + (channel ? N : 4); }
 
-// grid (64-row tiles x 2 chunks, heads)
-template <bool CHANNEL>
+// v_mfma_f32_16x16x4_f32: lane l holds A[l % 16][l / 16], B[l / 16][l % 16], D[4 (l / 16) + r][l % 16] in register r
+SYM_DEV f32x4 mfma4(float x, float y, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(x, y, c, 0, 0, 0); }
+SYM_DEV f32x4 lds4(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
+SYM_DEV f32x4 exp2_neg(f32x4 v) {       // 2^v for exponents that are <= 0 where they matter
+  f32x4 r;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) r[i] = __builtin_amdgcn_exp2f(fminf(v[i], 0.f));
+  return r;
+}
+
+// grid (64-row tiles x 2 chunks, heads); NN: 16-channel tiles (N <= 16 NN)
+template <bool CHANNEL, int NN>
 __global__ __launch_bounds__(NT) void delta_chunk_prep_kernel(DeltaRuleArgs a) {
   extern __shared__ float lds[];
-  const int N = a.N, N4 = (N + 3) & ~3, ld = N4 + 4;
+  constexpr int NP = 16 * NN, LD = NP + 4;
+  constexpr int TSTEP = NT / NP, EPT = C / TSTEP;      // a thread stages channel n of the tokens tt0, tt0 + TSTEP, ..
+  const int N = a.N;
   const int h = blockIdx.y, tile = blockIdx.x >> 1, sub = blockIdx.x & 1;
   const int seq = a.tiles[2 * tile], off = a.tiles[2 * tile + 1];
   const int q0 = a.cu_q[seq], qlen = a.cu_q[seq + 1] - q0;
@@ -205,26 +221,37 @@ __global__ __launch_bounds__(NT) void delta_chunk_prep_kernel(DeltaRuleArgs a) {
   const int nt = min(C, qlen - off - C * sub);
   if (nt <= 0) return;
   const long long r0 = q0 + off + C * sub;
-  float* kS = lds;                             // [C][ld]
-  float* qS = kS + C * ld;
-  float* GS = qS + C * ld;                     // CHANNEL: [C][ld], else [C]
-  float* LS = GS + (CHANNEL ? C * ld : C);     // [C][LC] beta_i Akk_ij below the diagonal
-  float* TS = LS + C * LC;                     // [C][LC]
-  float* bS = TS + C * LC;                     // [C]
-  const long long gn = (long long)a.G * N;
-  const float* q = a.q + (long long)(h / a.hpg) * N;
-  const float* k = a.k + (long long)(h / a.hpg) * N;
+  float* kS = lds;                             // [C][LD]
+  float* qS = kS + C * LD;                     // [C][LD]
+  float* GS = qS + C * LD;                     // CHANNEL: [C][LD], else [C]
+  float* XS = GS + (CHANNEL ? C * LD : C);     // [2 halves of the channels][Akk, Aqk][C][LC]
+  float* bS = XS + 4 * C * LC;                 // [C]
+  float* LS = XS;                              // afterwards: [C][LC] beta_i Akk_ij below the diagonal
+  float* TS = XS + 2 * C * LC;                 // [C][LC]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int n = tid % NP, tt0 = tid / NP;
+  const int gn = a.G * N;
   const float rate2 = expf(a.A_log[h]) * LOG2E;
-  const int tid = threadIdx.x;
-  for (int i = tid; i < C * N4; i += NT) {
-    const int tt = i / N4, n = i - tt * N4;
-    const bool in = tt < nt && n < N;
-    const long long r = r0 + tt;
-    kS[tt * ld + n] = in ? k[r * gn + n] : 0.f;
-    qS[tt * ld + n] = in ? q[r * gn + n] : 0.f;
-    if (CHANNEL)
-      GS[tt * ld + n] = in ? -rate2 * softplus_exact(a.dz[r * a.ldd + (long long)h * N + n] + a.dt_bias[(long long)h * N + n])
-                           : 0.f;
+  {
+    const float* k = a.k + (r0 + tt0) * gn + (h / a.hpg) * N + n;
+    const float* q = a.q + (r0 + tt0) * gn + (h / a.hpg) * N + n;
+    const float* dz = CHANNEL ? a.dz + (r0 + tt0) * a.ldd + h * N + n : nullptr;
+    const float db = CHANNEL && n < N ? a.dt_bias[h * N + n] : 0.f;
+    float rk[EPT], rq[EPT], rz[EPT];
+#pragma unroll
+    for (int u = 0; u < EPT; ++u) {
+      const bool in = tt0 + TSTEP * u < nt && n < N;
+      rk[u] = in ? k[(long long)TSTEP * u * gn] : 0.f;
+      rq[u] = in ? q[(long long)TSTEP * u * gn] : 0.f;
+      if (CHANNEL) rz[u] = in ? dz[TSTEP * u * a.ldd] : 0.f;
+    }
+#pragma unroll
+    for (int u = 0; u < EPT; ++u) {
+      const int o = (tt0 + TSTEP * u) * LD + n;
+      kS[o] = rk[u];
+      qS[o] = rq[u];
+      if (CHANNEL) GS[o] = tt0 + TSTEP * u < nt && n < N ? -rate2 * softplus_exact(rz[u] + db) : 0.f;
+    }
   }
   if (tid < C) {
     const bool in = tid < nt;
@@ -244,61 +271,118 @@ __global__ __launch_bounds__(NT) void delta_chunk_prep_kernel(DeltaRuleArgs a) {
   float* ws = a.ws + (r0 * a.H + h) * wc;      // row stride H * wc
   const long long wrow = (long long)a.H * wc;
   if (CHANNEL) {
-    for (int n = tid; n < N; n += NT) {
-      float g = 0.f;
-#pragma unroll 8
+    if (tid < NP) {
+      float g[C];
+#pragma unroll
+      for (int tt = 0; tt < C; ++tt) g[tt] = GS[tt * LD + tid];
+#pragma unroll
+      for (int tt = 1; tt < C; ++tt) g[tt] += g[tt - 1];
+#pragma unroll
       for (int tt = 0; tt < C; ++tt) {
-        g += GS[tt * ld + n];
-        GS[tt * ld + n] = g;
-        if (tt < nt) ws[tt * wrow + 2 * C + n] = g;
+        GS[tt * LD + tid] = g[tt];
+        if (tt < nt && tid < N) ws[tt * wrow + 2 * C + tid] = g[tt];
       }
     }
     __syncthreads();
   } else if (tid < nt) {
     ws[tid * wrow + 2 * C] = GS[tid];
   }
-  // scores of a 2 x 2 block of (i, j) per thread
-  const int ib = tid >> 4, jb = tid & 15;
-  float kk[2][2] = {{0.f, 0.f}, {0.f, 0.f}}, qk[2][2] = {{0.f, 0.f}, {0.f, 0.f}};
-  if (jb <= ib) {
-    for (int n = 0; n < N4; n += 4) {
-      float4 ki[2], qi[2], kj[2], gi[2], gj[2];
+  // scores.  A wave takes one half of the channels (half) of Akk or Aqk (kind) for the matrix products
+  constexpr int NH = NN > 1 ? NN / 2 : 1;      // 16-channel tiles per half
+  const int half = wave >> 1, kind = wave & 1;
+  const int col = lane & 15, g = lane >> 4;
+  {
+    const float* iS = kind ? qS : kS;
+    f32x4 d00 = {0.f, 0.f, 0.f, 0.f}, d10 = d00, d11 = d00;
+    if (NN > 1 || half == 0) {
 #pragma unroll
-      for (int e = 0; e < 2; ++e) {
-        ki[e] = *reinterpret_cast<const float4*>(kS + (2 * ib + e) * ld + n);
-        qi[e] = *reinterpret_cast<const float4*>(qS + (2 * ib + e) * ld + n);
-        kj[e] = *reinterpret_cast<const float4*>(kS + (2 * jb + e) * ld + n);
+      for (int t = 0; t < NH; ++t) {
+        const int c = 16 * (half * NH + t) + 4 * g;
+        f32x4 i1 = lds4(iS + (16 + col) * LD + c);
+        f32x4 j0 = lds4(kS + col * LD + c);
         if (CHANNEL) {
-          gi[e] = *reinterpret_cast<const float4*>(GS + (2 * ib + e) * ld + n);
-          gj[e] = *reinterpret_cast<const float4*>(GS + (2 * jb + e) * ld + n);
+          const f32x4 mid = lds4(GS + 15 * LD + c);
+          i1 = i1 * exp2_neg(lds4(GS + (16 + col) * LD + c) - mid);
+          j0 = j0 * exp2_neg(mid - lds4(GS + col * LD + c));
+#pragma unroll
+          for (int r = 0; r < 4; ++r) d10 = mfma4(i1[r], j0[r], d10);
+        } else {
+          const f32x4 i0 = lds4(iS + col * LD + c), j1 = lds4(kS + (16 + col) * LD + c);
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            d00 = mfma4(i0[r], j0[r], d00);
+            d10 = mfma4(i1[r], j0[r], d10);
+            d11 = mfma4(i1[r], j1[r], d11);
+          }
         }
       }
+    }
+    float* X = XS + (half * 2 + kind) * C * LC;
 #pragma unroll
-      for (int e = 0; e < 2; ++e)
-#pragma unroll
-        for (int f = 0; f < 2; ++f) {
-          float4 w = kj[f];
-          if (CHANNEL) {   // (entries above the diagonal: exponent clamped, never used)
-            w.x *= __builtin_amdgcn_exp2f(fminf(gi[e].x - gj[f].x, 0.f));
-            w.y *= __builtin_amdgcn_exp2f(fminf(gi[e].y - gj[f].y, 0.f));
-            w.z *= __builtin_amdgcn_exp2f(fminf(gi[e].z - gj[f].z, 0.f));
-            w.w *= __builtin_amdgcn_exp2f(fminf(gi[e].w - gj[f].w, 0.f));
-          }
-          kk[e][f] += ki[e].x * w.x + ki[e].y * w.y + ki[e].z * w.z + ki[e].w * w.w;
-          qk[e][f] += qi[e].x * w.x + qi[e].y * w.y + qi[e].z * w.z + qi[e].w * w.w;
-        }
+    for (int r = 0; r < 4; ++r) {
+      X[(16 + 4 * g + r) * LC + col] = d10[r];
+      if (!CHANNEL) {
+        X[(4 * g + r) * LC + col] = d00[r];
+        X[(16 + 4 * g + r) * LC + 16 + col] = d11[r];
+      }
     }
   }
+  if (CHANNEL) {
+    // diagonal tiles: wave (half, tile), a 2 x 2 block of (i, j) per lane, both kinds
+    const int dt = wave & 1, ib = lane >> 3, jb = lane & 7;
+    const int i0 = 16 * dt + 2 * ib, j0 = 16 * dt + 2 * jb;
+    float kk[2][2] = {{0.f, 0.f}, {0.f, 0.f}}, qk[2][2] = {{0.f, 0.f}, {0.f, 0.f}};
+    if (jb <= ib && (NN > 1 || half == 0)) {
+#pragma unroll 2
+      for (int c = 16 * NH * half; c < 16 * NH * (half + 1); c += 4) {
+        f32x4 ki[2], qi[2], kj[2], gi[2], gj[2];
 #pragma unroll
-  for (int e = 0; e < 2; ++e)
+        for (int e = 0; e < 2; ++e) {
+          ki[e] = lds4(kS + (i0 + e) * LD + c);
+          qi[e] = lds4(qS + (i0 + e) * LD + c);
+          gi[e] = lds4(GS + (i0 + e) * LD + c);
+          kj[e] = lds4(kS + (j0 + e) * LD + c);
+          gj[e] = lds4(GS + (j0 + e) * LD + c);
+        }
 #pragma unroll
-    for (int f = 0; f < 2; ++f) {
-      const int i = 2 * ib + e, j = 2 * jb + f;
-      float w = 1.f;
-      if (!CHANNEL) w = __builtin_amdgcn_exp2f(fminf(GS[i] - GS[j], 0.f));
-      LS[i * LC + j] = j < i ? bS[i] * kk[e][f] * w : 0.f;
-      if (i < nt) ws[i * wrow + C + j] = j <= i ? qk[e][f] * w : 0.f;
+        for (int e = 0; e < 2; ++e)
+#pragma unroll
+          for (int f = 0; f < 2; ++f) {
+            const f32x4 w = kj[f] * exp2_neg(gi[e] - gj[f]);    // (above the diagonal: clamped, never used)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+              kk[e][f] += ki[e][r] * w[r];
+              qk[e][f] += qi[e][r] * w[r];
+            }
+          }
+      }
     }
+    float* X = XS + half * 2 * C * LC;
+#pragma unroll
+    for (int e = 0; e < 2; ++e)
+#pragma unroll
+      for (int f = 0; f < 2; ++f) {
+        X[(i0 + e) * LC + j0 + f] = kk[e][f];
+        X[C * LC + (i0 + e) * LC + j0 + f] = qk[e][f];
+      }
+  }
+  __syncthreads();
+  // the halves meet; Akk goes on as beta_i Akk_ij (the threads hold their sums across a barrier: LS lies on XS)
+  float lv[C * C / NT];
+#pragma unroll
+  for (int u = 0; u < C * C / NT; ++u) {
+    const int i = (tid + NT * u) / C, j = (tid + NT * u) % C;
+    const int o = i * LC + j;
+    float w = 1.f;
+    if (!CHANNEL) w = __builtin_amdgcn_exp2f(fminf(GS[i] - GS[j], 0.f));
+    const bool stored = !(i < 16 && j >= 16);
+    lv[u] = j < i ? bS[i] * w * (XS[o] + XS[2 * C * LC + o]) : 0.f;
+    const float av = stored && j <= i ? w * (XS[C * LC + o] + XS[3 * C * LC + o]) : 0.f;
+    if (i < nt) ws[i * wrow + C + j] = av;
+  }
+  __syncthreads();
+#pragma unroll
+  for (int u = 0; u < C * C / NT; ++u) LS[(tid + NT * u) / C * LC + (tid + NT * u) % C] = lv[u];
   __syncthreads();
   // T = (I + L)^-1 diag(beta): thread c solves column c by forward substitution
   if (tid < C) {
@@ -317,131 +401,156 @@ __global__ __launch_bounds__(NT) void delta_chunk_prep_kernel(DeltaRuleArgs a) {
     }
   }
   __syncthreads();
-  for (int i = tid; i < C * C; i += NT) {
-    const int tt = i / C, c = i - tt * C;
-    if (tt < nt) ws[tt * wrow + c] = TS[tt * LC + c];
+#pragma unroll
+  for (int u = 0; u < C * C / NT; ++u) {
+    const int i = (tid + NT * u) / C, c = (tid + NT * u) % C;
+    if (i < nt) ws[i * wrow + c] = TS[i * LC + c];
   }
 }
 
-// v_mfma_f32_16x16x4_f32: lane l holds A[l % 16][l / 16], B[l / 16][l % 16], D[4 (l / 16) + r][l % 16] in register r
-SYM_DEV f32x4 mfma4(float x, float y, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(x, y, c, 0, 0, 0); }
-
-// grid (P / 64, heads, runs); NN: 16-row tiles of the state (N <= 16 NN)
-template <typename T, bool CHANNEL, int NN>
-__global__ __launch_bounds__(NT) void delta_chunk_scan_kernel(DeltaRuleArgs a) {
+// grid (P / 64, heads, runs), 512 threads: waves 0 .. 3 multiply (16 value columns each), waves 4 .. 7 stage.  NN: 16-row
+// tiles of the state (N <= 16 NN); NBUF: LDS stages (two where they fit)
+template <typename T, bool CHANNEL, int NN, int NBUF>
+__global__ __launch_bounds__(2 * NT) void delta_chunk_scan_kernel(DeltaRuleArgs a) {
   extern __shared__ float lds[];
   constexpr int NP = 16 * NN;                  // padded key channels
   constexpr int LD = NP + 4;
-  constexpr int EPT = C * NP / NT;             // staged (token, channel) entries per thread
+  constexpr int TSTEP = NT / NP, EPT = C / TSTEP;      // a staging thread owns channel n of the tokens tt0, tt0 + TSTEP, ..
+  constexpr int oQ = C * LD, oH = 2 * C * LD, oT = oH + NP * LC, oA = oT + C * LC, oD = oA + C * LC, STAGE = oD + NP;
   const int N = a.N, P = a.P;
   const int h = blockIdx.y, run = blockIdx.z;
   const int s0 = a.cu_q[run], s1 = a.cu_q[run + 1];
   if (s1 <= s0) return;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int chunks = (s1 - s0 + C - 1) / C;
+  const int wc = ws_cols(CHANNEL, N);
+  const long long wrow = (long long)a.H * wc;
+  if (wave >= 4) {
+    // ---- staging waves -----------------------------------------------------------------------------------------
+    const int tid = threadIdx.x - NT, n = tid % NP, tt0 = tid / NP;
+    const bool nin = n < N;
+    const int gn = a.G * N;
+    const float* k = a.k + (long long)(s0 + tt0) * gn + (h / a.hpg) * N + n;
+    const float* q = a.q + (long long)(s0 + tt0) * gn + (h / a.hpg) * N + n;
+    const float* wsh = a.ws + (long long)s0 * wrow + (long long)h * wc;
+    const float* G = wsh + tt0 * wrow + 2 * C + (CHANNEL ? n : 0);
+    const int mj = tid % C, mt = tid / C;      // the [C][C] matrices: column mj of the rows mt, mt + NT / C, ..
+    const float* M = wsh + mt * wrow + mj;
+    constexpr int MSTEP = NT / C, MPT = C / MSTEP;
+    // a chunk waits in registers until its stage is free; at sizes where that does not fit (one stage), it is loaded a few
+    // rows at a time instead
+    constexpr bool AHEAD = NBUF == 2;
+    constexpr int EB = AHEAD ? EPT : 4;
+    float rk[EB], rq[EB], rg[EB], gl, rt[MPT], ra[MPT];
+    auto fetch = [&](int c, int u0) {
+      const int t0 = c * C, nt = min(C, s1 - s0 - t0);
+      const float* kc = k + (long long)t0 * gn;
+      const float* qc = q + (long long)t0 * gn;
+      const float* Gc = G + t0 * wrow;
+#pragma unroll
+      for (int e = 0; e < EB; ++e) {
+        const int u = u0 + e;
+        const bool row = tt0 + TSTEP * u < nt;
+        rk[e] = row && nin ? kc[(long long)TSTEP * u * gn] : 0.f;
+        rq[e] = row && nin ? qc[(long long)TSTEP * u * gn] : 0.f;
+        rg[e] = row && (nin || !CHANNEL) ? Gc[TSTEP * u * wrow] : 0.f;
+      }
+      if (u0) return;
+      gl = nin || !CHANNEL ? wsh[(long long)(t0 + nt - 1) * wrow + 2 * C + (CHANNEL ? n : 0)] : 0.f;
+      const float* Mc = M + t0 * wrow;
+#pragma unroll
+      for (int u = 0; u < MPT; ++u) {
+        const bool in = mt + MSTEP * u < nt && mj < nt;
+        rt[u] = in ? Mc[MSTEP * u * wrow] : 0.f;
+        ra[u] = in ? Mc[MSTEP * u * wrow + C] : 0.f;
+      }
+    };
+    auto put = [&](float* st, int u0) {
+#pragma unroll
+      for (int e = 0; e < EB; ++e) {
+        const int tt = tt0 + TSTEP * (u0 + e);
+        const float eg = __builtin_amdgcn_exp2f(rg[e]);
+        st[tt * LD + n] = rk[e] * eg;
+        st[oQ + tt * LD + n] = rq[e] * eg;
+        st[oH + n * LC + tt] = rk[e] * __builtin_amdgcn_exp2f(fminf(gl - rg[e], 0.f));   // (rows past the run's end: k = 0)
+      }
+    };
+    auto stash = [&](float* st, int c) {
+      if (AHEAD) {
+        put(st, 0);
+      } else {
+#pragma unroll 1
+        for (int u0 = 0; u0 < EPT; u0 += EB) {
+          fetch(c, u0);
+          put(st, u0);
+        }
+      }
+      if (tt0 == 0) st[oD + n] = __builtin_amdgcn_exp2f(gl);
+#pragma unroll
+      for (int u = 0; u < MPT; ++u) {
+        st[oT + (mt + MSTEP * u) * LC + mj] = rt[u];
+        st[oA + (mt + MSTEP * u) * LC + mj] = ra[u];
+      }
+    };
+    if (AHEAD) fetch(0, 0);
+    stash(lds, 0);
+    if (AHEAD && chunks > 1) fetch(1, 0);
+    __syncthreads();                           // chunk 0 is staged
+    for (int c = 0; c < chunks; ++c) {
+      if (NBUF == 1) __syncthreads();          // chunk c has been read
+      if (c + 1 < chunks) {
+        stash(lds + (NBUF == 2 ? ((c + 1) & 1) * STAGE : 0), c + 1);
+        if (AHEAD && c + 2 < chunks) fetch(c + 2, 0);
+      }
+      __syncthreads();                         // chunk c + 1 is staged (two stages: and chunk c has been read)
+    }
+    return;
+  }
+  // ---- multiplying waves -----------------------------------------------------------------------------------------
   const int col = lane & 15, g = lane >> 4;
   const int p = blockIdx.x * 64 + wave * 16 + col;
   const bool pin = p < P;
-  float* Kt = lds;                             // [C][LD]  k e^G
-  float* Qt = Kt + C * LD;                     // [C][LD]  q e^G
-  float* Kh = Qt + C * LD;                     // [NP][LC] k e^(G_C - G), channel-major
-  float* Tm = Kh + NP * LC;                    // [C][LC]
-  float* Aq = Tm + C * LC;                     // [C][LC]
-  float* D = Aq + C * LC;                      // [NP]     G_C
-  const long long gn = (long long)a.G * N;
-  const float* q = a.q + (long long)(h / a.hpg) * N;
-  const float* k = a.k + (long long)(h / a.hpg) * N;
-  const T* v = reinterpret_cast<const T*>(a.v) + (long long)h * P + p;
-  const int wc = ws_cols(CHANNEL, N);
-  const float* wsh = a.ws + (long long)h * wc;
-  const long long wrow = (long long)a.H * wc;
   const int pr = a.prev_row[s0];
   const int sv = a.save_slot[s1 - 1];
-  float rk[EPT], rq[EPT], rg[EPT], rt[C * C / NT], ra[C * C / NT], vn[8];
-  float rgl[CHANNEL ? (NP + NT - 1) / NT : 1];   // G of the chunk's last token
-  auto fetch = [&](int t0) {
-    const int nt = min(C, s1 - t0);
-#pragma unroll
-    for (int u = 0; u < EPT; ++u) {
-      const int i = tid + NT * u;
-      const int tt = i / NP, n = i % NP;
-      const bool in = tt < nt && n < N;
-      const long long r = t0 + tt;
-      rk[u] = in ? k[r * gn + n] : 0.f;
-      rq[u] = in ? q[r * gn + n] : 0.f;
-      if (CHANNEL) rg[u] = in ? wsh[r * wrow + 2 * C + n] : 0.f;
-      else rg[u] = tt < nt ? wsh[r * wrow + 2 * C] : 0.f;
-    }
-    const float* last = wsh + (long long)(t0 + nt - 1) * wrow + 2 * C;
-    if (CHANNEL) {
-#pragma unroll
-      for (int u = 0; u < (NP + NT - 1) / NT; ++u) {
-        const int n = tid + NT * u;
-        rgl[u] = n < N ? last[n] : 0.f;
-      }
-    } else {
-      rgl[0] = last[0];
-    }
-#pragma unroll
-    for (int u = 0; u < C * C / NT; ++u) {
-      const int i = tid + NT * u, tt = i / C, j = i % C;
-      const bool in = tt < nt && j < nt;
-      rt[u] = in ? wsh[(long long)(t0 + tt) * wrow + j] : 0.f;
-      ra[u] = in ? wsh[(long long)(t0 + tt) * wrow + C + j] : 0.f;
-    }
+  const long long hp = (long long)a.H * P;
+  const T* v = reinterpret_cast<const T*>(a.v) + (long long)s0 * hp + (long long)h * P + p;
+  float* out = a.out + (long long)s0 * hp + (long long)h * P + p;
+  float vn[8];
+  auto fetch_v = [&](int c) {
+    const int nt = min(C, s1 - s0 - c * C);
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const int tt = 16 * (i >> 2) + 4 * g + (i & 3);
-      vn[i] = tt < nt && pin ? (float)v[(long long)(t0 + tt) * a.H * P] : 0.f;
+      vn[i] = tt < nt && pin ? (float)v[(long long)(c * C + tt) * hp] : 0.f;
     }
   };
   f32x4 S[NN];
   const bool old = pr <= -2 && pin;
-  const float* st = a.state + (old ? (long long)(-(pr + 2)) * a.state_stride + (long long)h * N * P + p : 0);
+  const float* st0 = a.state + (old ? (long long)(-(pr + 2)) * a.state_stride + (long long)h * N * P + p : 0);
 #pragma unroll
   for (int t = 0; t < NN; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int n = 16 * t + 4 * g + r;
-      S[t][r] = old && n < N ? st[(long long)n * P] : 0.f;
+      S[t][r] = old && n < N ? st0[(long long)n * P] : 0.f;
     }
-  fetch(s0);
-  for (int t0 = s0; t0 < s1; t0 += C) {
-    const int nt = min(C, s1 - t0);
-    __syncthreads();   // everyone is done with the previous chunk
-    // G of the last token first: the entries' exponents need it
-    if (CHANNEL) {
-#pragma unroll
-      for (int u = 0; u < (NP + NT - 1) / NT; ++u)
-        if (tid + NT * u < NP) D[tid + NT * u] = rgl[u];
-      __syncthreads();
-    }
-#pragma unroll
-    for (int u = 0; u < EPT; ++u) {
-      const int i = tid + NT * u;
-      const int tt = i / NP, n = i % NP;
-      const float gl = CHANNEL ? D[n] : rgl[0];
-      const float eg = __builtin_amdgcn_exp2f(rg[u]);
-      Kt[tt * LD + n] = rk[u] * eg;
-      Qt[tt * LD + n] = rq[u] * eg;
-      Kh[n * LC + tt] = rk[u] * __builtin_amdgcn_exp2f(fminf(gl - rg[u], 0.f));   // (rows past the run's end: k = 0)
-    }
-#pragma unroll
-    for (int u = 0; u < C * C / NT; ++u) {
-      const int i = tid + NT * u, tt = i / C, j = i % C;
-      Tm[tt * LC + j] = rt[u];
-      Aq[tt * LC + j] = ra[u];
-    }
-    f32x4 V0 = {vn[0], vn[1], vn[2], vn[3]}, V1 = {vn[4], vn[5], vn[6], vn[7]};
-    const float dh = CHANNEL ? 0.f : __builtin_amdgcn_exp2f(rgl[0]);
-    __syncthreads();
-    if (t0 + C < s1) fetch(t0 + C);
+  fetch_v(0);
+  __syncthreads();                             // chunk 0 is staged
+  for (int c = 0; c < chunks; ++c) {
+    const float* st = lds + (NBUF == 2 ? (c & 1) * STAGE : 0);
+    const float* Kt = st + col * LD + 4 * g;
+    const float* Qt = st + oQ + col * LD + 4 * g;
+    const float* Kh = st + oH + col * LC + 4 * g;
+    const float* Tm = st + oT + col * LC + 4 * g;
+    const float* Aq = st + oA + col * LC + 4 * g;
+    const float* D = st + oD + 4 * g;
+    const f32x4 V0 = {vn[0], vn[1], vn[2], vn[3]}, V1 = {vn[4], vn[5], vn[6], vn[7]};
+    if (c + 1 < chunks) fetch_v(c + 1);
     f32x4 K0 = {0.f, 0.f, 0.f, 0.f}, K1 = K0, O0 = K0, O1 = K0;
 #pragma unroll
     for (int t = 0; t < NN; ++t) {
-      const f32x4 x0 = *reinterpret_cast<const f32x4*>(Kt + col * LD + 16 * t + 4 * g);
-      const f32x4 x1 = *reinterpret_cast<const f32x4*>(Kt + (16 + col) * LD + 16 * t + 4 * g);
-      const f32x4 y0 = *reinterpret_cast<const f32x4*>(Qt + col * LD + 16 * t + 4 * g);
-      const f32x4 y1 = *reinterpret_cast<const f32x4*>(Qt + (16 + col) * LD + 16 * t + 4 * g);
+      const f32x4 x0 = lds4(Kt + 16 * t), x1 = lds4(Kt + 16 * LD + 16 * t);
+      const f32x4 y0 = lds4(Qt + 16 * t), y1 = lds4(Qt + 16 * LD + 16 * t);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         K0 = mfma4(x0[r], S[t][r], K0);
@@ -453,9 +562,7 @@ __global__ __launch_bounds__(NT) void delta_chunk_scan_kernel(DeltaRuleArgs a) {
     const f32x4 R0 = V0 - K0, R1 = V1 - K1;
     f32x4 U0 = {0.f, 0.f, 0.f, 0.f}, U1 = U0;
     {
-      const f32x4 x00 = *reinterpret_cast<const f32x4*>(Tm + col * LC + 4 * g);
-      const f32x4 x10 = *reinterpret_cast<const f32x4*>(Tm + (16 + col) * LC + 4 * g);
-      const f32x4 x11 = *reinterpret_cast<const f32x4*>(Tm + (16 + col) * LC + 16 + 4 * g);
+      const f32x4 x00 = lds4(Tm), x10 = lds4(Tm + 16 * LC), x11 = lds4(Tm + 16 * LC + 16);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         U0 = mfma4(x00[r], R0[r], U0);
@@ -465,9 +572,7 @@ __global__ __launch_bounds__(NT) void delta_chunk_scan_kernel(DeltaRuleArgs a) {
       for (int r = 0; r < 4; ++r) U1 = mfma4(x11[r], R1[r], U1);
     }
     {
-      const f32x4 x00 = *reinterpret_cast<const f32x4*>(Aq + col * LC + 4 * g);
-      const f32x4 x10 = *reinterpret_cast<const f32x4*>(Aq + (16 + col) * LC + 4 * g);
-      const f32x4 x11 = *reinterpret_cast<const f32x4*>(Aq + (16 + col) * LC + 16 + 4 * g);
+      const f32x4 x00 = lds4(Aq), x10 = lds4(Aq + 16 * LC), x11 = lds4(Aq + 16 * LC + 16);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         O0 = mfma4(x00[r], U0[r], O0);
@@ -477,32 +582,26 @@ __global__ __launch_bounds__(NT) void delta_chunk_scan_kernel(DeltaRuleArgs a) {
       for (int r = 0; r < 4; ++r) O1 = mfma4(x11[r], U1[r], O1);
     }
 #pragma unroll
-    for (int t = 0; t < NN; ++t) {
-      if (CHANNEL) {
-        const f32x4 d = *reinterpret_cast<const f32x4*>(D + 16 * t + 4 * g);
-#pragma unroll
-        for (int r = 0; r < 4; ++r) S[t][r] *= __builtin_amdgcn_exp2f(d[r]);
-      } else {
-        S[t] = S[t] * dh;
-      }
-    }
+    for (int t = 0; t < NN; ++t) S[t] = S[t] * lds4(D + 16 * t);
 #pragma unroll
     for (int t = 0; t < NN; ++t) {
-      const f32x4 x0 = *reinterpret_cast<const f32x4*>(Kh + (16 * t + col) * LC + 4 * g);
-      const f32x4 x1 = *reinterpret_cast<const f32x4*>(Kh + (16 * t + col) * LC + 16 + 4 * g);
+      const f32x4 x0 = lds4(Kh + 16 * t * LC), x1 = lds4(Kh + 16 * t * LC + 16);
 #pragma unroll
       for (int r = 0; r < 4; ++r) S[t] = mfma4(x0[r], U0[r], S[t]);
 #pragma unroll
       for (int r = 0; r < 4; ++r) S[t] = mfma4(x1[r], U1[r], S[t]);
     }
     if (pin) {
+      const int nt = min(C, s1 - s0 - c * C);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int i0 = 4 * g + r, i1 = 16 + i0;
-        if (i0 < nt) a.out[((long long)(t0 + i0) * a.H + h) * P + p] = O0[r];
-        if (i1 < nt) a.out[((long long)(t0 + i1) * a.H + h) * P + p] = O1[r];
+        if (i0 < nt) out[(long long)(c * C + i0) * hp] = O0[r];
+        if (i1 < nt) out[(long long)(c * C + i1) * hp] = O1[r];
       }
     }
+    if (NBUF == 1) __syncthreads();            // chunk c has been read
+    __syncthreads();                           // chunk c + 1 is staged (two stages: and chunk c has been read)
   }
   if (sv >= 0 && pin) {
     float* so = a.state + (long long)sv * a.state_stride + (long long)h * N * P + p;
@@ -548,29 +647,30 @@ void serial(const DeltaRuleArgs& a, hipStream_t s) {
 }
 
 template <typename T, bool CHANNEL, int NN>
-void launch_scan(const DeltaRuleArgs& a, hipStream_t s) {
-  constexpr int NP = 16 * NN;
-  const size_t lds = (size_t)(2 * C * (NP + 4) + NP * LC + 2 * C * LC + NP) * sizeof(float);
+void launch_chunks(const DeltaRuleArgs& a, hipStream_t s) {
+  constexpr int NP = 16 * NN, LD = NP + 4;
+  constexpr int STAGE = 2 * C * LD + NP * LC + 2 * C * LC + NP;
+  constexpr int NBUF = 2 * STAGE * (int)sizeof(float) <= 160 * 1024 ? 2 : 1;
+  const size_t prep = (size_t)((CHANNEL ? 3 : 2) * C * LD + 4 * C * LC + 2 * C) * sizeof(float);
+  const size_t scan = (size_t)NBUF * STAGE * sizeof(float);
   static bool raised = false;
-  if (!raised && lds > 64 * 1024) raise_lds(reinterpret_cast<const void*>(&delta_chunk_scan_kernel<T, CHANNEL, NN>));
-  raised = true;
-  delta_chunk_scan_kernel<T, CHANNEL, NN><<<dim3((a.P + 63) / 64, a.H, a.runs), NT, lds, s>>>(a);
+  if (!raised) {
+    raise_lds(reinterpret_cast<const void*>(&delta_chunk_prep_kernel<CHANNEL, NN>));
+    raise_lds(reinterpret_cast<const void*>(&delta_chunk_scan_kernel<T, CHANNEL, NN, NBUF>));
+    raised = true;
+  }
+  delta_chunk_prep_kernel<CHANNEL, NN><<<dim3(2 * a.ntiles, a.H), NT, prep, s>>>(a);
+  delta_chunk_scan_kernel<T, CHANNEL, NN, NBUF><<<dim3((a.P + 63) / 64, a.H, a.runs), 2 * NT, scan, s>>>(a);
 }
 
 template <typename T, bool CHANNEL>
 void chunked(const DeltaRuleArgs& a, hipStream_t s) {
-  const int ld = ((a.N + 3) & ~3) + 4;
-  const size_t lds = (size_t)(2 * C * ld + (CHANNEL ? C * ld : C) + 2 * C * LC + C) * sizeof(float);
-  static bool raised = false;
-  if (!raised) raise_lds(reinterpret_cast<const void*>(&delta_chunk_prep_kernel<CHANNEL>));
-  raised = true;
-  delta_chunk_prep_kernel<CHANNEL><<<dim3(2 * a.ntiles, a.H), NT, lds, s>>>(a);
   const int nn = (a.N + 15) / 16;
-  if (nn <= 1) launch_scan<T, CHANNEL, 1>(a, s);
-  else if (nn <= 2) launch_scan<T, CHANNEL, 2>(a, s);
-  else if (nn <= 4) launch_scan<T, CHANNEL, 4>(a, s);
-  else if (nn <= 8) launch_scan<T, CHANNEL, 8>(a, s);
-  else launch_scan<T, CHANNEL, 16>(a, s);
+  if (nn <= 1) launch_chunks<T, CHANNEL, 1>(a, s);
+  else if (nn <= 2) launch_chunks<T, CHANNEL, 2>(a, s);
+  else if (nn <= 4) launch_chunks<T, CHANNEL, 4>(a, s);
+  else if (nn <= 8) launch_chunks<T, CHANNEL, 8>(a, s);
+  else launch_chunks<T, CHANNEL, 16>(a, s);
 }
 
 }  // namespace

@@ -330,19 +330,122 @@ __global__ __launch_bounds__(BT) void residual_layer_norm_kernel(ResidualLnArgs 
   }
 }
 
-// A wave per (ROWS consecutive rows, head of q | k | v); a lane owns VC neighbouring channels of the head, PER times over
-// (64 VC PER >= the widest head).  VC = 4: eight- or sixteen-byte accesses (row strides, head sizes and bases permitting).
+// One head's share of conv_silu_qkv: which channels of the projection a unit covers, and where its row goes
+struct ConvUnit {
+  int kind, hd, width, c0;     // kind 0: q, 1: k, 2: v
+};
+SYM_DEV ConvUnit conv_unit(const ConvSiluArgs& a, int unit) {
+  ConvUnit u;
+  u.kind = unit < a.G ? 0 : (unit < 2 * a.G ? 1 : 2);
+  u.hd = unit - u.kind * a.G;
+  u.width = u.kind == 2 ? a.P : a.N;
+  u.c0 = u.kind * a.G * a.N + u.hd * u.width;
+  return u;
+}
+
+// silu, unit length (q, k), store.  y: the wave's PER x VC convolved channels of the row's head
+template <typename T, int VC, int PER>
+SYM_DEV void conv_silu_store(const ConvSiluArgs& a, const ConvUnit& un, int row, int lane, float (&y)[PER][VC]) {
+  float sq = 0.f;
+#pragma unroll
+  for (int u = 0; u < PER; ++u)
+#pragma unroll
+    for (int i = 0; i < VC; ++i) {
+      y[u][i] *= sigmoidf(y[u][i]);      // (channels past the head's width are 0)
+      sq += y[u][i] * y[u][i];
+    }
+  float r = 1.f;
+  if (un.kind < 2) r = 1.f / sqrtf(wave_sum(sq) + a.eps) * (un.kind == 0 ? a.q_scale : 1.f);
+#pragma unroll
+  for (int u = 0; u < PER; ++u) {
+    const int e = VC * (lane + 64 * u);
+    if (e < un.width) {
+      if (un.kind < 2) {
+        float* o = (un.kind == 0 ? a.q_out : a.k_out) + (long long)row * a.G * a.N + un.hd * un.width + e;
+        if constexpr (VC == 4) st4(o, make_float4(y[u][0] * r, y[u][1] * r, y[u][2] * r, y[u][3] * r));
+        else o[0] = y[u][0] * r;
+      } else {
+        T* o = reinterpret_cast<T*>(a.v_out) + ((long long)row * a.H + un.hd) * un.width + e;
+        if constexpr (VC == 4) st4(o, make_float4(y[u][0], y[u][1], y[u][2], y[u][3]));
+        else o[0] = (T)y[u][0];
+      }
+    }
+  }
+}
+
+// The usual tap counts, heads up to 256 wide, four channels per lane: the taps are loaded once per wave and the inputs
+// slide through registers from row to row (a run's start reloads them from the slot).  A wave per (ROWS rows, head).
+template <typename T, int TAPS, int ROWS>
+__global__ void conv_silu_qkv_taps_kernel(ConvSiluArgs a) {
+  const int lane = threadIdx.x & 63;
+  const int unit = blockIdx.y * (blockDim.x >> 6) + (threadIdx.x >> 6);
+  if (unit >= 2 * a.G + a.H) return;
+  const ConvUnit un = conv_unit(a, unit);
+  const int C = a.C, e = 4 * lane, c = un.c0 + e;
+  const bool in = e < un.width;
+  const T* z = reinterpret_cast<const T*>(a.z);
+  T wr[4 * TAPS];              // [channel][tap]
+  if (in) {
+    const T* w = reinterpret_cast<const T*>(a.w) + (long long)c * TAPS;
+#pragma unroll
+    for (int i = 0; i < TAPS; ++i)
+      __builtin_memcpy(wr + 4 * i, __builtin_assume_aligned(w + 4 * i, 4 * sizeof(T)), 4 * sizeof(T));
+  }
+  T hist[TAPS][4];             // hist[b]: the input b places back
+  int run0 = -1;
+  const int r0 = blockIdx.x * ROWS, r1 = min(a.T, r0 + ROWS);
+  for (int row = r0; row < r1; ++row) {
+    const int s0 = a.cu_q ? a.cu_q[a.row_seq[row]] : row;
+    float y[1][4] = {{0.f, 0.f, 0.f, 0.f}};
+    if (in) {
+      if (s0 != run0) {
+        const int j = row - s0;
+        const int pr = j < TAPS - 1 ? a.prev_row[s0] : -1;
+        const T* st = pr <= -2 ? reinterpret_cast<const T*>(a.state) + (long long)(-(pr + 2)) * a.state_stride : nullptr;
+#pragma unroll
+        for (int b = 1; b < TAPS; ++b) {
+          const T* src = b <= j ? z + (long long)(row - b) * a.ldz + c : (st ? st + (long long)(TAPS - 1 - (b - j)) * C + c : nullptr);
+          if (src) {
+            __builtin_memcpy(hist[b], __builtin_assume_aligned(src, 4 * sizeof(T)), 4 * sizeof(T));
+          } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) hist[b][i] = (T)0.f;
+          }
+        }
+      } else {
+#pragma unroll
+        for (int b = TAPS - 1; b > 0; --b)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) hist[b][i] = hist[b - 1][i];
+      }
+      __builtin_memcpy(hist[0], __builtin_assume_aligned(z + (long long)row * a.ldz + c, 4 * sizeof(T)), 4 * sizeof(T));
+#pragma unroll
+      for (int b = 0; b < TAPS; ++b)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) y[0][i] += (float)wr[i * TAPS + TAPS - 1 - b] * (float)hist[b][i];
+      // (as in the general kernel: a row that is a run of its own moves the carried taps on)
+      if (!a.cu_q && a.save_slot && a.save_slot[row] >= 0) {
+        T* dst = reinterpret_cast<T*>(a.state) + (long long)a.save_slot[row] * a.state_stride;
+#pragma unroll
+        for (int b = 0; b < TAPS - 1; ++b)
+          __builtin_memcpy(__builtin_assume_aligned(dst + (long long)(TAPS - 2 - b) * C + c, 4 * sizeof(T)), hist[b],
+                           4 * sizeof(T));
+      }
+    }
+    run0 = s0;
+    conv_silu_store<T, 4, 1>(a, un, row, lane, y);
+  }
+}
+
+// Any tap count: a wave per (ROWS consecutive rows, head); a lane owns VC neighbouring channels of the head, PER times
+// over (64 VC PER >= the widest head).  VC = 4: eight- or sixteen-byte accesses (strides, head sizes and bases permitting).
 template <typename T, int VC, int PER, int ROWS>
 __global__ void conv_silu_qkv_kernel(ConvSiluArgs a) {
   const int lane = threadIdx.x & 63;
   const int unit = blockIdx.y * (blockDim.x >> 6) + (threadIdx.x >> 6);
   if (unit >= 2 * a.G + a.H) return;
   const int taps = a.taps, C = a.C, keep = taps - 1;
-  const int nq = a.G * a.N;
-  const int kind = unit < a.G ? 0 : (unit < 2 * a.G ? 1 : 2);     // q, k or v head
-  const int hd = unit - kind * a.G;
-  const int width = kind == 2 ? a.P : a.N;
-  const int c0 = kind * nq + hd * width;
+  const ConvUnit un = conv_unit(a, unit);
   const T* z = reinterpret_cast<const T*>(a.z);
   const T* w = reinterpret_cast<const T*>(a.w);
   for (int row = blockIdx.x * ROWS; row < min(a.T, (int)(blockIdx.x + 1) * ROWS); ++row) {
@@ -353,14 +456,13 @@ __global__ void conv_silu_qkv_kernel(ConvSiluArgs a) {
     const int sv = (!a.cu_q && a.save_slot) ? a.save_slot[row] : -1;
     T* dst = sv >= 0 && keep ? reinterpret_cast<T*>(a.state) + (long long)sv * a.state_stride : nullptr;
     float y[PER][VC];
-    float sq = 0.f;
 #pragma unroll
     for (int u = 0; u < PER; ++u) {
       const int e = VC * (lane + 64 * u);
 #pragma unroll
       for (int i = 0; i < VC; ++i) y[u][i] = 0.f;
-      if (e < width) {
-        const int c = c0 + e;
+      if (e < un.width) {
+        const int c = un.c0 + e;
         T hist[MAX_TAPS][VC];     // hist[b]: the input b places back (b = 0: this row's)
 #pragma unroll
         for (int b = 0; b < MAX_TAPS; ++b) {
@@ -380,11 +482,6 @@ __global__ void conv_silu_qkv_kernel(ConvSiluArgs a) {
           if (b < taps)
 #pragma unroll
             for (int i = 0; i < VC; ++i) y[u][i] += (float)w[(long long)(c + i) * taps + keep - b] * (float)hist[b][i];
-#pragma unroll
-        for (int i = 0; i < VC; ++i) {
-          y[u][i] *= sigmoidf(y[u][i]);
-          sq += y[u][i] * y[u][i];
-        }
         // rows that are runs of their own: this lane alone reads and writes its channels of the row's slot, so the carried
         // taps move on here (place m holds the input keep - m back from the next token)
         if (dst) {
@@ -398,23 +495,7 @@ __global__ void conv_silu_qkv_kernel(ConvSiluArgs a) {
         }
       }
     }
-    float r = 1.f;
-    if (kind < 2) r = 1.f / sqrtf(wave_sum(sq) + a.eps) * (kind == 0 ? a.q_scale : 1.f);
-#pragma unroll
-    for (int u = 0; u < PER; ++u) {
-      const int e = VC * (lane + 64 * u);
-      if (e < width) {
-        if (kind < 2) {
-          float* o = (kind == 0 ? a.q_out : a.k_out) + (long long)row * nq + hd * width + e;
-          if constexpr (VC == 4) st4(o, make_float4(y[u][0] * r, y[u][1] * r, y[u][2] * r, y[u][3] * r));
-          else o[0] = y[u][0] * r;
-        } else {
-          T* o = reinterpret_cast<T*>(a.v_out) + ((long long)row * a.H + hd) * width + e;
-          if constexpr (VC == 4) st4(o, make_float4(y[u][0], y[u][1], y[u][2], y[u][3]));
-          else o[0] = (T)y[u][0];
-        }
-      }
-    }
+    conv_silu_store<T, VC, PER>(a, un, row, lane, y);
   }
 }
 
@@ -504,23 +585,30 @@ void launch_residual_layer_norm(const ResidualLnArgs& a, int f32, hipStream_t s)
 #undef LN
 }
 
-template <int VC, int PER>
-static void conv_silu_rows(const ConvSiluArgs& a, int f32, hipStream_t s) {
-  const int units = 2 * a.G + a.H;
-  if (a.T <= 256) {
-    DISPATCH_T(f32, (conv_silu_qkv_kernel<T, VC, PER, 1><<<dim3(a.T, units), 64, 0, s>>>(a));)
-  } else {
-    DISPATCH_T(f32, (conv_silu_qkv_kernel<T, VC, PER, 4><<<dim3((a.T + 3) / 4, (units + 3) / 4), 256, 0, s>>>(a));)
+// grid of a kernel with a wave per (rows, head): decode-sized launches one row and one wave per workgroup
+#define CONV_ROWS(KERNEL1, KERNELN, ROWS)                                                                     \
+  if (a.T <= 256) {                                                                                           \
+    DISPATCH_T(f32, (KERNEL1<<<dim3(a.T, units), 64, 0, s>>>(a));)                                            \
+  } else {                                                                                                    \
+    DISPATCH_T(f32, (KERNELN<<<dim3((a.T + ROWS - 1) / ROWS, (units + 3) / 4), 256, 0, s>>>(a));)             \
   }
-}
 
 void launch_conv_silu_qkv(const ConvSiluArgs& a, int f32, hipStream_t s) {
   if (a.T <= 0) return;
   const auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
-  const int wide = a.N > a.P ? a.N : a.P;
-  const bool vec = a.N % 4 == 0 && a.P % 4 == 0 && a.ldz % 4 == 0 && al(a.z) && al(a.state) && a.state_stride % 4 == 0 &&
-                   al(a.q_out) && al(a.k_out) && al(a.v_out);
-  if (vec && wide <= 256) conv_silu_rows<4, 1>(a, f32, s);
-  else if (vec) conv_silu_rows<4, 2>(a, f32, s);      // heads up to 512 wide (checked by the op layer)
-  else conv_silu_rows<1, 8>(a, f32, s);
+  const int wide = a.N > a.P ? a.N : a.P, units = 2 * a.G + a.H;
+  const bool vec = a.N % 4 == 0 && a.P % 4 == 0 && a.ldz % 4 == 0 && al(a.z) && al(a.w) && al(a.state) &&
+                   a.state_stride % 4 == 0 && al(a.q_out) && al(a.k_out) && al(a.v_out);
+  if (vec && wide <= 256 && a.taps == 4) {
+    CONV_ROWS((conv_silu_qkv_taps_kernel<T, 4, 1>), (conv_silu_qkv_taps_kernel<T, 4, 8>), 8)
+  } else if (vec && wide <= 256 && a.taps == 3) {
+    CONV_ROWS((conv_silu_qkv_taps_kernel<T, 3, 1>), (conv_silu_qkv_taps_kernel<T, 3, 8>), 8)
+  } else if (vec && wide <= 256 && a.taps == 2) {
+    CONV_ROWS((conv_silu_qkv_taps_kernel<T, 2, 1>), (conv_silu_qkv_taps_kernel<T, 2, 8>), 8)
+  } else if (vec) {      // heads up to 512 wide (checked by the op layer)
+    CONV_ROWS((conv_silu_qkv_kernel<T, 4, 2, 1>), (conv_silu_qkv_kernel<T, 4, 2, 4>), 4)
+  } else {
+    CONV_ROWS((conv_silu_qkv_kernel<T, 1, 8, 1>), (conv_silu_qkv_kernel<T, 1, 8, 4>), 4)
+  }
 }
+#undef CONV_ROWS
