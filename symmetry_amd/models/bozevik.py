@@ -133,7 +133,7 @@ class BozevikLM:
             "gq": t("mix.dq.norm"), "gkv": t("mix.dkv.norm") if owner else None,
             "uq": t("mix.uq"),
             "uk": t("mix.uk").view(m.heads, m.dim, m.kv_rank),                     # [H, dn, r]: q_n @ uk[h]
-            "uvt": t("mix.uv").view(m.heads, m.vdim, m.kv_rank).transpose(1, 2),   # [H, r, dv] view
+            "uvt": t("mix.uv").view(m.heads, m.vdim, m.kv_rank).transpose(1, 2).contiguous(),   # [H, r, dv]
             "o": t("mix.o"), "rope": self._rope_table(m, max_pos),
         }
         if isinstance(layer.mlp, GluSpec):
@@ -270,12 +270,7 @@ class BozevikLM:
         xn = self._buf(name + ".xn", (n, cfg.hidden_size))
         ops.layer_norm(x, rows, self.final_norm, cfg.norm_eps, xn)
         logits = self._buf(name, (n, cfg.vocab_size), torch.float32)
-        if self.dtype == torch.float32:
-            torch.matmul(xn, self.embed.t(), out=logits)
-        elif self.device.type == "cpu":
-            logits.copy_(xn.float() @ self.embed.float().t())
-        else:
-            torch.bmm(xn[None], self.embed.t()[None], out_dtype=torch.float32, out=logits[None])
+        ops.linear_f32(xn, self.embed, logits)
         if cfg.logit_scale != 1.0:
             logits.mul_(cfg.logit_scale)
         return logits

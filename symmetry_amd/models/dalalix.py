@@ -196,14 +196,7 @@ class DalalixLM:
 
     def _linear_f32(self, name: str, x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
         """x [R, K] @ w[N, K]^T -> fp32 [R, N] (the library GEMM's fp32 accumulator, unrounded)."""
-        out = self._buf(name, (x.shape[0], w.shape[0]), torch.float32)
-        if self.dtype == torch.float32:
-            torch.matmul(x, w.t(), out=out)
-        elif self.device.type == "cpu":
-            out.copy_(x.float() @ w.float().t())
-        else:
-            torch.bmm(x[None], w.t()[None], out_dtype=torch.float32, out=out[None])
-        return out
+        return ops.linear_f32(x, w, self._buf(name, (x.shape[0], w.shape[0]), torch.float32))
 
     @staticmethod
     def _cols(z: torch.Tensor, P: dict, name: str) -> torch.Tensor:

@@ -159,7 +159,7 @@ class KomazenLM:
             P["gq"], P["gkv"] = t("mix.dq.norm"), t("mix.dkv.norm") if owner else None
             P["uq"] = t("mix.uq")
             P["uk"] = t("mix.uk").view(m.heads, m.dim, m.kv_rank)                     # [H, dn, r]: q_n @ uk[h]
-            P["uvt"] = t("mix.uv").view(m.heads, m.vdim, m.kv_rank).transpose(1, 2)   # [H, r, dv] view
+            P["uvt"] = t("mix.uv").view(m.heads, m.vdim, m.kv_rank).transpose(1, 2).contiguous()   # [H, r, dv]
             P["rope"] = self._rope_table(m, max_pos)
         else:
             if m.vdim > 512:
@@ -301,10 +301,5 @@ class KomazenLM:
         xn = self._buf(name + ".xn", (n, cfg.hidden_size))
         ops.rms_norm_rows(x, rows, self.final_norm, cfg.norm_eps, 0.0, xn)
         logits = self._buf(name, (n, cfg.vocab_size), torch.float32)
-        if self.dtype == torch.float32:
-            torch.matmul(xn, self.head.t(), out=logits)
-        elif self.device.type == "cpu":
-            logits.copy_(xn.float() @ self.head.float().t())
-        else:
-            torch.bmm(xn[None], self.head.t()[None], out_dtype=torch.float32, out=logits[None])
+        ops.linear_f32(xn, self.head, logits)
         return logits

@@ -347,10 +347,5 @@ class LemunexLM:
         xn = self._buf(name + ".xn", (n, cfg.hidden_size))
         ops.rms_norm_rows(x, rows, self.final_norm, cfg.norm_eps, NORM_OFFSET, xn)
         logits = self._buf(name, (n, cfg.vocab_size), torch.float32)
-        if self.dtype == torch.float32:
-            torch.matmul(xn, self.head.t(), out=logits)
-        elif self.device.type == "cpu":
-            logits.copy_(xn.float() @ self.head.float().t())
-        else:
-            torch.bmm(xn[None], self.head.t()[None], out_dtype=torch.float32, out=logits[None])
+        ops.linear_f32(xn, self.head, logits)
         return logits
