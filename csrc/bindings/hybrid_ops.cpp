@@ -829,7 +829,8 @@ void residual_layer_norm(Tensor& x, const OptTensor& base, const OptTensor& a, c
 
 void conv_silu_qkv(const Tensor& z, const Tensor& w, Tensor& state, const OptTensor& cu_q, const OptTensor& row_seq,
                    const Tensor& prev_row, const OptTensor& save_slot, int64_t runs, int64_t G, int64_t N, int64_t H,
-                   int64_t P, double q_scale, double unit_eps, Tensor& q_out, Tensor& k_out, Tensor& v_out) {
+                   int64_t P, double q_scale, double unit_eps, Tensor& q_out, Tensor& k_out, Tensor& v_out, const OptTensor& gx,
+                   const OptTensor& gw, const OptTensor& gout) {
   const int f32 = act(w, "w");
   TORCH_CHECK(z.dim() == 2 && w.dim() == 2 && state.dim() == 3, "conv_silu_qkv: z [T, C], w [C, taps], state [slots, taps - 1, C]");
   const int64_t T = z.size(0), C = 2 * G * N + H * P, taps = w.size(1);
@@ -869,6 +870,18 @@ void conv_silu_qkv(const Tensor& z, const Tensor& w, Tensor& state, const OptTen
   a.q_scale = (float)q_scale;
   a.eps = (float)unit_eps;
   a.T = (int)T, a.C = (int)C, a.taps = (int)taps, a.G = (int)G, a.N = (int)N, a.H = (int)H, a.P = (int)P;
+  if (gx.has_value()) {
+    TORCH_CHECK(gw.has_value() && gout.has_value() && T <= 256, "conv_silu_qkv: the extra projection needs its weight and output, at most 256 rows");
+    TORCH_CHECK(gw->dim() == 2 && gout->numel() == T * gw->size(0) && 2 * G + H + gw->size(0) <= 65535, "conv_silu_qkv: projection shapes");
+    same_act(*gw, f32, "gw");
+    dtype(*gout, at::kFloat, "gout");
+    a.ldgx = view2(*gx, f32, T, gw->size(1), "gx");
+    a.gx = gx->data_ptr();
+    a.gw = gw->data_ptr();
+    a.gout = ptr<float>(*gout);
+    a.gn = (int)gw->size(0);
+    a.gd = (int)gw->size(1);
+  }
   launch_conv_silu_qkv(a, f32, cur_stream(z));
 }
 
@@ -1017,7 +1030,7 @@ TORCH_LIBRARY(symmetry_amd_hybrid, m) {
   m.def(
       "conv_silu_qkv(Tensor z, Tensor w, Tensor(a!) state, Tensor? cu_q, Tensor? row_seq, Tensor prev_row, Tensor? save_slot, "
       "int runs, int G, int N, int H, int P, float q_scale, float unit_eps, Tensor(b!) q_out, Tensor(c!) k_out, "
-      "Tensor(d!) v_out) -> ()",
+      "Tensor(d!) v_out, Tensor? gx=None, Tensor? gw=None, Tensor(e!)? gout=None) -> ()",
       &conv_silu_qkv);
   m.def(
       "delta_rule(bool channel, Tensor q, Tensor k, Tensor v, Tensor dz, Tensor dt_bias, Tensor A_log, Tensor bz, "

@@ -293,6 +293,11 @@ struct ConvSiluArgs {
   void* v_out;          // [T][H][P] activation dtype
   float q_scale, eps;
   int T, C, taps, G, N, H, P;
+  // optional, decode-sized steps (T <= 256): gout [T][gn] = gx . gw[j] in fp32 (waves of their own in the same launch)
+  const void* gx; long long ldgx;
+  const void* gw;       // [gn][gd] activation dtype
+  float* gout;
+  int gn, gd;
 };
 void launch_conv_silu_qkv(const ConvSiluArgs& a, int f32, hipStream_t s);
 // x = cap tanh(x / cap)

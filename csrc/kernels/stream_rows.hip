@@ -12,12 +12,13 @@
 //   residual_layer_norm  x = base + a + b on the fp32 stream and the next sublayer's layer norm (weight, bias) from the same
 //                        pass; also the gathered norm in front of the output head
 //   conv_silu_qkv        causal per-channel convolution of q | k | v with carried taps, silu, unit-vector q / k heads (a wave
-//                        per (rows, head))
+//                        per (rows, head)); in decode-sized steps also a few fp32 projections of the same input
 //
 // One workgroup per row unless noted; columns strided over the threads (coalesced), any width.  All statistics, mixing
 // and sums are fp32; only the stored activations take the activation dtype T (bf16 or float).
 #include "common.h"
 #include "hybrid_launchers.h"
+#include "wave_dot.h"
 
 namespace {
 
@@ -373,13 +374,25 @@ SYM_DEV void conv_silu_store(const ConvSiluArgs& a, const ConvUnit& un, int row,
   }
 }
 
+// A wave past the heads: one output of the small projection that rides along (one row per wave)
+template <typename T>
+SYM_DEV void conv_gate_unit(const ConvSiluArgs& a, int j, int row, int lane) {
+  if (j >= a.gn) return;
+  const float v = wave_dot<T>(reinterpret_cast<const T*>(a.gx) + (long long)row * a.ldgx,
+                              reinterpret_cast<const T*>(a.gw) + (long long)j * a.gd, a.gd, lane);
+  if (lane == 0) a.gout[(long long)row * a.gn + j] = v;
+}
+
 // The usual tap counts, heads up to 256 wide, four channels per lane: the taps are loaded once per wave and the inputs
 // slide through registers from row to row (a run's start reloads them from the slot).  A wave per (ROWS rows, head).
 template <typename T, int TAPS, int ROWS>
 __global__ void conv_silu_qkv_taps_kernel(ConvSiluArgs a) {
   const int lane = threadIdx.x & 63;
   const int unit = blockIdx.y * (blockDim.x >> 6) + (threadIdx.x >> 6);
-  if (unit >= 2 * a.G + a.H) return;
+  if (unit >= 2 * a.G + a.H) {
+    if (ROWS == 1 && a.gn) conv_gate_unit<T>(a, unit - 2 * a.G - a.H, blockIdx.x, lane);
+    return;
+  }
   const ConvUnit un = conv_unit(a, unit);
   const int C = a.C, e = 4 * lane, c = un.c0 + e;
   const bool in = e < un.width;
@@ -443,7 +456,10 @@ template <typename T, int VC, int PER, int ROWS>
 __global__ void conv_silu_qkv_kernel(ConvSiluArgs a) {
   const int lane = threadIdx.x & 63;
   const int unit = blockIdx.y * (blockDim.x >> 6) + (threadIdx.x >> 6);
-  if (unit >= 2 * a.G + a.H) return;
+  if (unit >= 2 * a.G + a.H) {
+    if (ROWS == 1 && a.gn) conv_gate_unit<T>(a, unit - 2 * a.G - a.H, blockIdx.x, lane);
+    return;
+  }
   const int taps = a.taps, C = a.C, keep = taps - 1;
   const ConvUnit un = conv_unit(a, unit);
   const T* z = reinterpret_cast<const T*>(a.z);
@@ -588,7 +604,7 @@ void launch_residual_layer_norm(const ResidualLnArgs& a, int f32, hipStream_t s)
 // grid of a kernel with a wave per (rows, head): decode-sized launches one row and one wave per workgroup
 #define CONV_ROWS(KERNEL1, KERNELN, ROWS)                                                                     \
   if (a.T <= 256) {                                                                                           \
-    DISPATCH_T(f32, (KERNEL1<<<dim3(a.T, units), 64, 0, s>>>(a));)                                            \
+    DISPATCH_T(f32, (KERNEL1<<<dim3(a.T, units + a.gn), 64, 0, s>>>(a));)                                          \
   } else {                                                                                                    \
     DISPATCH_T(f32, (KERNELN<<<dim3((a.T + ROWS - 1) / ROWS, (units + 3) / 4), 256, 0, s>>>(a));)             \
   }

@@ -112,7 +112,7 @@ def build_kernels(verbose: bool = False, force: bool = False) -> str:
     kdir = os.path.join(CSRC, "kernels")
     # (the family libraries' launcher headers are not included by these translation units)
     headers = [h for h in glob.glob(os.path.join(kdir, "*.h")) + glob.glob(os.path.join(kdir, "*.cuh"))
-               if os.path.basename(h) not in ("latent_launchers.h", "hybrid_launchers.h")]
+               if os.path.basename(h) not in ("latent_launchers.h", "hybrid_launchers.h", "wave_dot.h")]
     sources = sorted(s for s in glob.glob(os.path.join(kdir, "*.hip"))
                      if os.path.basename(s) not in LATENT_KERNELS + HYBRID_KERNELS)
     tinc, tlib, abi = _torch_paths()
@@ -188,7 +188,7 @@ def build_hybrid(verbose: bool = False, force: bool = False) -> str:
     symmetry_amd/_C_hybrid.so (``torch.ops.symmetry_amd_hybrid``)."""
     os.makedirs(OBJ, exist_ok=True)
     kdir = os.path.join(CSRC, "kernels")
-    headers = [os.path.join(kdir, h) for h in ("common.h", "hybrid_launchers.h", "latent_launchers.h")]
+    headers = [os.path.join(kdir, h) for h in ("common.h", "wave_dot.h", "hybrid_launchers.h", "latent_launchers.h")]
     tinc, tlib, abi = _torch_paths()
     jobs, objs = [], []
     for name in HYBRID_KERNELS + HYBRID_SHARED:

@@ -27,8 +27,8 @@ Caches and states belong to a layer RUN: a looped layer has one plane or one sta
 that reads a sublayer's input is one row block of one fused weight (a single library GEMM), except the recurrence's step
 sizes and decays, whose GEMMs leave their fp32 accumulator unrounded; the kernels take column ranges as views.  Step
 launches per layer run: GEMM (the mixer's projections), then
-    delta:   GEMM W_b | W_a (fp32; channel decays: W_b, W_a2), conv_silu_qkv (+ conv_state_update in prompt steps),
-             delta_rule, (GEMM W_g2,) gated_group_norm, GEMM W_o
+    delta:   GEMM W_b | W_a (fp32; channel decays: W_b, W_a2), conv_silu_qkv (+ conv_state_update in prompt steps; in
+             decode steps W_b | W_a ride along in this launch), delta_rule, (GEMM W_g2,) gated_group_norm, GEMM W_o
     latent:  latent_prep, bmm (absorb W_uk), rope_pairs, latent_attn (sink, gate), bmm (W_uv), GEMM W_o
     residual_layer_norm; GEMM gate|up, silu_mul, GEMM down; residual_layer_norm (+ e in front of a loop's next pass)
 All intermediates live in the preallocated Workspace, so decode steps are hipGraph-capturable.
@@ -47,6 +47,7 @@ from .lemunex import _Fused
 from .transformer import MAX_STEP_SEQS, ForwardBatch, Workspace
 from .weights import ModelWeights
 
+GATES_ALONG_ROWS = 64  # decode steps up to this many rows compute beta / decay pre-activations beside the convolution
 UNIT_EPS = 1e-6       # inside the root of the queries' and keys' length (fixed by the design)
 
 
@@ -191,14 +192,20 @@ class BeletarLM:
         prefill = b.kind != "decode"
         cu = b.cu_q if prefill else None
         z = self._linear("z", h, P["w_h"])
-        gates = self._linear_f32("del.gates", h, P["gates"])
+        # (a decode step's few rows take these few outputs along in the convolution's launch)
+        along = None
+        if not prefill and T <= GATES_ALONG_ROWS:
+            gates = self._buf("del.gates", (T, P["gates"].shape[0]), torch.float32)
+            along = (h, P["gates"], gates)
+        else:
+            gates = self._linear_f32("del.gates", h, P["gates"])
         dz = self._linear_f32("del.dz", self._cols(z, P, "a1"), P["a2"]) if m.channel else gates[:, H:]
         qkv = self._cols(z, P, "qkv")
         f32 = torch.float32
         q, k = self._buf("del.q", (T, G, N), f32), self._buf("del.k", (T, G, N), f32)
         v = self._buf("del.v", (T, H, V))
         ops.conv_silu_qkv(qkv, P["conv"], cache.conv[n], cu, b.row_seq, b.prev_row, runs, G, N, H, V, N ** -0.5, UNIT_EPS,
-                          q, k, v, save_slot=None if prefill else b.save_slot)
+                          q, k, v, save_slot=None if prefill else b.save_slot, gates=along)
         if prefill and m.conv > 1:
             ops.conv_state_update(qkv, cache.conv[n], cu, b.prev_row, b.save_slot, runs)
         y = self._buf("del.y", (T, H * V), f32)

@@ -1040,15 +1040,19 @@ def residual_layer_norm(x, a=None, b=None, w=None, bias=None, eps=0.0, rows=None
 
 
 def conv_silu_qkv(z, w, state, cu_q, row_seq, prev_row, runs, G, N, H, P, q_scale, unit_eps, q_out, k_out, v_out,
-                  save_slot=None):
+                  save_slot=None, gates=None):
     """z [T, G N | G N | H P] (a view) = q | k | v through the causal per-channel convolution w [C, taps] over every run
     (inputs before a run from state[slot] [taps - 1, C] where prev_row[first] <= -2, else zero), then silu; q and k heads
     (N entries) become unit vectors y / sqrt(sum y^2 + unit_eps), q also times q_scale -> q_out, k_out fp32 [T, G, N]; v ->
     v_out [T, H, P].  ``save_slot`` with cu_q None (every row its own run): the launch moves the row's carried taps on
-    itself; otherwise conv_state_update follows."""
+    itself; otherwise conv_state_update follows.  ``gates`` = (x [T, d], w [n, d], out fp32 [T, n]): out = x w^T in the same
+    launch, for a projection of a few outputs on decode-sized steps (T <= 256)."""
     if _gpu(z):
         return _hyb().conv_silu_qkv(z, w, state, cu_q, row_seq if cu_q is not None else None, prev_row, save_slot, int(runs),
-                                    int(G), int(N), int(H), int(P), float(q_scale), float(unit_eps), q_out, k_out, v_out)
+                                    int(G), int(N), int(H), int(P), float(q_scale), float(unit_eps), q_out, k_out, v_out,
+                                    *(gates or ()))
+    if gates is not None:
+        linear_f32(*gates)
     reference.conv_silu_qkv(z, w, state, cu_q, prev_row, runs, G, N, H, P, q_scale, unit_eps, q_out, k_out, v_out)
     if save_slot is not None and state.shape[1]:
         reference.conv_state_update(z, state, cu_q, prev_row, save_slot, runs)

@@ -545,8 +545,12 @@ def test_convolved_projections_with_carried_taps(device, taps, shape):
         q, k, v = torch.empty(T, G, N), torch.empty(T, G, N), torch.empty(T, H, P)
         z, q, k, v, prev, save, rs, cu = _dev(device, z, q, k, v, prev, save, rs, cu)
         zin = z[:, :C_]
-        if decode:
-            ops.conv_silu_qkv(zin, wd, state, None, None, prev, T, G, N, H, P, 0.3, 1e-6, q, k, v, save_slot=save)
+        if decode:      # (with a small projection of another input in the same launch)
+            x, gw = torch.randn(T, 70), torch.randn(5, 66)
+            xd, gwd, go = _dev(device, x, gw, torch.empty(T, 5))
+            ops.conv_silu_qkv(zin, wd, state, None, None, prev, T, G, N, H, P, 0.3, 1e-6, q, k, v, save_slot=save,
+                              gates=(xd[:, :66], gwd, go))
+            assert float((go.cpu().double() - x[:, :66].double() @ gw.double().T).abs().max()) < 1e-4
         else:
             ops.conv_silu_qkv(zin, wd, state, cu, rs, prev, runs, G, N, H, P, 0.3, 1e-6, q, k, v)
             if taps > 1:
