@@ -134,7 +134,8 @@ class LLMEngine:
         if cfg.dtype not in ("bfloat16", "float32"):
             raise ValueError(f"dtype {cfg.dtype!r}: bfloat16 or float32")
         dtype = torch.float32 if cfg.dtype == "float32" else torch.bfloat16
-        if dtype == torch.float32 and not getattr(cls, "has_seq_state", False):
+        f32_capable = getattr(cls, "has_seq_state", False) or getattr(cls, "serves_float32", False)
+        if dtype == torch.float32 and not f32_capable:
             raise ValueError(f"{mcfg.name}: this model family is served in bfloat16 only")
         if cfg.weights == "random":
             mode = cfg.weight_init
@@ -150,7 +151,7 @@ class LLMEngine:
         self._kv_elem = 4 if dtype == torch.float32 else 2
         per_block = mcfg.kv_bytes_per_token(self._kv_elem) // cfg.tp_size * cfg.block_size
         kv_need = (cfg.num_kv_blocks or -(-cfg.max_num_seqs * max_model_len // cfg.block_size)) * per_block
-        extra = {"dtype": dtype} if getattr(cls, "has_seq_state", False) else {}
+        extra = {"dtype": dtype} if f32_capable else {}
         self.model = cls(weights, self.device, tp_comm=tp_comm, ep_comm=ep_comm, max_decode_ctx=max_model_len,
                          decode_weights=cfg.decode_weights, kv_reserve_bytes=kv_need, **extra)
         self.tokenizer = load_tokenizer(mcfg, cfg.tokenizer or (cfg.weights if cfg.weights != "random" else None))

@@ -157,7 +157,9 @@ class ModelRunner:
         self.ctx_blocks = [b for b in self.ctx_blocks if b <= self.max_blocks]
         self.is_gpu = self.device.type != "cpu"
         self.use_graphs = use_graphs and self.is_gpu
-        self.seq_state = bool(getattr(model, "has_seq_state", False))
+        # the packed metadata carries previous rows / state slots / row -> sequence (models without state slots that ask
+        # for the row map get "none" for the first two)
+        self.seq_state = bool(getattr(model, "has_seq_state", False) or getattr(model, "row_metadata", False))
         # pad short prefills to the graph buckets (without use_graphs -- CPU tests -- they then run eagerly)
         self.prefill_graphs = self.use_graphs
         self.prefill_graph_replays = 0

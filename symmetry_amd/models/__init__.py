@@ -23,6 +23,10 @@ def model_class(cfg):
         from .beletar import BeletarLM
 
         return BeletarLM
+    if family == "bekedra":
+        from .bekedra import BekedraLM
+
+        return BekedraLM
     if family == "llama":
         from .transformer import TransformerLM
 

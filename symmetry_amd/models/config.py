@@ -278,6 +278,10 @@ class RotarySpec:
     fast: float = 0.0
     slow: float = 0.0
     half: bool = False           # True: entry i turns with entry i + dims / 2 (half layout) instead of the pairs (2i, 2i + 1)
+    # scaling by wavelength instead of ``fast`` / ``slow`` (set both): waves shorter than original / high keep their
+    # frequency, waves longer than original / low are divided by ``factor``, a linear blend between; no magnitude
+    low: float = 0.0
+    high: float = 0.0
 
 
 @dataclass(frozen=True)
@@ -1220,6 +1224,222 @@ SMALL_BELETAR = beletar_stack("small-beletar", 32768, 2048, "DCCL", heads=8, kv_
                               att_heads=16, embed_scale=8.0, scaling=(4.0, 4096.0, 32.0, 1.0), max_position=8192,
                               bos_token_id=32000, eos_token_ids=(32001, 32002))
 
+# --------------------------------------------------------------------------------------------------
+# Bekedra: parallel layers (one RMS norm feeds the mixer and the routed feed-forward, both added to the stream) listed one
+# by one, a range of them run several times in a row with the same weights (a learned vector per pass added in front of every
+# pass, caches per pass); mixers: softmax attention whose values are its projected keys (norms over whole projections, query
+# temperature, no rotation), or per-head normed half-layout rotary attention with soft-capped scores, a sink and an
+# element-wise output gate; squared-ReLU experts, softmax over the chosen logits; logits through the embedding table.
+# --------------------------------------------------------------------------------------------------
+@dataclass(frozen=True)
+class NormedAttnSpec:
+    """Causal softmax attention with normed queries and keys and grouped key / value heads; every mechanism off by default."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    row_norm: bool = False       # norms over the whole query / key projection (else per head, one weight for all heads)
+    bias: bool = False           # q / k projections carry biases
+    key_values: bool = False     # the values are the projected keys before their norm (vdim == dim, no value projection)
+    temp_coef: float = 0.0       # queries times 1 + temp_coef ln(floor((p + 1) / temp_every) + 1) at position p
+    temp_every: int = 1
+    rot: RotarySpec | None = None
+    softcap: float = 0.0         # scores through softcap tanh(s / softcap); 0: none
+    sink: bool = False           # a learned per-head logit in the softmax's denominator (no key, no value)
+    gate: bool = False           # concatenated heads times sigmoid(W_g h), element by element
+
+
+@dataclass(frozen=True)
+class ChosenSoftmaxSpec:
+    """Router with biased logits: the ``top`` largest, weights = softmax over the chosen ones; squared-ReLU experts."""
+    experts: int
+    top: int
+    expert_ff: int
+
+
+@dataclass(frozen=True)
+class BekedraLayer:
+    type: str                    # "attention" | "attention_2"
+    mixer: NormedAttnSpec
+    mlp: ChosenSoftmaxSpec | None = None
+
+
+@dataclass(frozen=True)
+class BekedraConfig:
+    family = "bekedra"
+    name: str
+    vocab_size: int
+    hidden_size: int
+    layers: tuple
+    loop: LoopSpec | None = None
+    embed_scale: float = 1.0
+    norm_eps: float = 1e-5
+    max_position: int = 131072
+    bos_token_id: int = 1
+    eos_token_ids: tuple = (2,)
+    chat_format: str = "llama3"
+    tie_embeddings = True
+    rope_scaling = None
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def is_moe(self) -> bool:
+        return any(layer.mlp is not None for layer in self.layers)
+
+    def layer_runs(self) -> list:
+        """The layers in the order they run: (layer, number of the loop's pass that starts with it, else None).  Caches
+        belong to the entries of this list."""
+        n, lp = len(self.layers), self.loop
+        if lp is None:
+            return [(i, None) for i in range(n)]
+        out = [(i, None) for i in range(lp.start)]
+        for t in range(lp.times):
+            out += [(i, t if i == lp.start else None) for i in range(lp.start, lp.stop)]
+        return out + [(i, None) for i in range(lp.stop, n)]
+
+    def num_params(self) -> int:
+        from .weights import bekedra_shapes
+
+        n = 0
+        for shape in bekedra_shapes(self).values():
+            k = 1
+            for v in shape:
+                k *= v
+            n += k
+        return n
+
+    def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
+        """(key-value layers keep one plane and an fp32 key scale per token)"""
+        n = 0
+        for i, _ in self.layer_runs():
+            m = self.layers[i].mixer
+            n += m.kv_heads * m.dim * dtype_bytes + (4 if m.key_values else m.kv_heads * m.vdim * dtype_bytes)
+        return n
+
+    def replace(self, **kw) -> "BekedraConfig":
+        return dataclasses.replace(self, **kw)
+
+
+def _wave_scaling(scaling, where: str) -> dict:
+    if not scaling:
+        return {}
+    factor, low, high, orig = _take(scaling, where, "factor", "low", "high", "original")
+    return {"factor": float(factor), "original": float(orig), "low": float(low), "high": float(high)}
+
+
+def bekedra_from_config(cfg: dict, name: str = "bekedra") -> BekedraConfig:
+    """config.json of a Bekedra checkpoint: every size and constant is read here; a key this reader does not know means a
+    mechanism this code does not have, so it raises."""
+    layers = []
+    for i, L in enumerate(cfg["layers"]):
+        kind, mixer, mlp = _take(L, f"layer {i}", "type", "mixer", optional=("mlp",))
+        if kind == "attention":
+            dim, heads, kvh, temp, scale, vdim = _take(mixer, f"layer {i} mixer", "dim", "heads", "kv_heads", "q_temp",
+                                                       "scale", "vdim")
+            coef, every = _take(temp, f"layer {i} q_temp", "coef", "every")
+            mix = NormedAttnSpec(int(heads), int(kvh), int(dim), int(vdim), float(scale), row_norm=True, bias=True,
+                                 key_values=True, temp_coef=float(coef), temp_every=int(every))
+            if mix.vdim != mix.dim or mix.temp_every < 1 or mix.temp_every != every:
+                raise ValueError(f"layer {i}: vdim {vdim} / dim {dim} / q_temp.every {every} do not fit")
+        elif kind == "attention_2":
+            dim, heads, kvh, rot, scale, cap, vdim = _take(mixer, f"layer {i} mixer", "dim", "heads", "kv_heads", "rot",
+                                                           "scale", "softcap", "vdim")
+            base, dims, scaling = _take(rot, f"layer {i} rot", "base", "dims", optional=("scaling",))
+            rspec = RotarySpec(int(dims), float(base), half=True, **_wave_scaling(scaling, f"layer {i} rot.scaling"))
+            mix = NormedAttnSpec(int(heads), int(kvh), int(dim), int(vdim), float(scale), rot=rspec, softcap=float(cap),
+                                 sink=True, gate=True)
+            if rspec.dims % 2 or rspec.dims > mix.dim or mix.softcap <= 0:
+                raise ValueError(f"layer {i}: rot.dims {dims} / dim {dim} / softcap {cap} do not fit")
+        else:
+            raise ValueError(f"layer {i}: unknown layer type {kind!r}")
+        if mix.heads % mix.kv_heads:
+            raise ValueError(f"layer {i}: heads {heads} / kv_heads {kvh} do not fit")
+        if mlp is None:
+            ff = None
+        elif mlp.get("kind") == "moe":
+            _, exp, router = _take(mlp, f"layer {i} mlp", "kind", "expert", "router")
+            (eff,) = _take(exp, f"layer {i} mlp.expert", "ff")
+            experts, top = _take(router, f"layer {i} mlp.router", "experts", "top")
+            ff = ChosenSoftmaxSpec(int(experts), int(top), int(eff))
+            if not 1 <= ff.top <= ff.experts:
+                raise ValueError(f"layer {i}: top {top} of {experts} experts")
+        else:
+            raise ValueError(f"layer {i}: unknown mlp kind {mlp.get('kind')!r}")
+        layers.append(BekedraLayer(kind, mix, ff))
+    vocab, width, norm, _, emb, loop, _, bos, eos = _take(
+        cfg, "config", "vocab", "width", "norm", "layers", "embedding",
+        optional=("loop", "architecture", "bos_token_id", "eos_token_ids"))
+    (eps,) = _take(norm, "norm", "eps")
+    (escale,) = _take(emb, "embedding", "scale")
+    if loop:
+        loop = LoopSpec(*(int(v) for v in _take(loop, "loop", "start", "stop", "times")))
+        if not 0 <= loop.start < loop.stop <= len(layers) or loop.times < 1:
+            raise ValueError(f"loop {loop}: not a range of the {len(layers)} layers")
+    return BekedraConfig(name=name, vocab_size=int(vocab), hidden_size=int(width), layers=tuple(layers), loop=loop or None,
+                         embed_scale=float(escale), norm_eps=float(eps), bos_token_id=int(bos if bos is not None else 1),
+                         eos_token_ids=tuple(eos) if eos is not None else (2,))
+
+
+def bekedra_to_config(c: BekedraConfig) -> dict:
+    """The config.json form of a BekedraConfig (exports, tests)."""
+    layers = []
+    for layer in c.layers:
+        m = layer.mixer
+        md = {"dim": m.dim, "heads": m.heads, "kv_heads": m.kv_heads, "scale": m.scale, "vdim": m.vdim}
+        if layer.type == "attention":
+            md["q_temp"] = {"coef": m.temp_coef, "every": m.temp_every}
+        else:
+            md["rot"], md["softcap"] = {"base": m.rot.base, "dims": m.rot.dims}, m.softcap
+            if m.rot.factor > 0:
+                md["rot"]["scaling"] = {"factor": m.rot.factor, "high": m.rot.high, "low": m.rot.low,
+                                        "original": m.rot.original}
+        f = layer.mlp
+        fd = None if f is None else {"expert": {"ff": f.expert_ff}, "kind": "moe",
+                                     "router": {"experts": f.experts, "top": f.top}}
+        layers.append({"mixer": md, "mlp": fd, "type": layer.type})
+    out = {"architecture": "Bekedra", "embedding": {"scale": c.embed_scale}, "layers": layers, "norm": {"eps": c.norm_eps},
+           "vocab": c.vocab_size, "width": c.hidden_size}
+    if c.loop:
+        out["loop"] = {"start": c.loop.start, "stop": c.loop.stop, "times": c.loop.times}
+    return out
+
+
+def bekedra_stack(name, vocab, width, pattern, heads, kv_heads, dim, experts, top, expert_ff, rot_dims=None, vdim=None,
+                  rot_heads=None, rot_kv_heads=None, rot_dim=None, loop=None, embed_scale=1.0, scaling=(8.0, 1.0, 4.0, 4096.0),
+                  softcap=50.0, temp=(0.1, 1024), **kw) -> BekedraConfig:
+    """A stack from a pattern string: "K" attention whose values are its keys, "R" rotary attention with soft cap, sink and
+    gate; lower case = no feed-forward.  ``loop`` = (start, stop, times), ``scaling`` = (factor, low, high, original)."""
+    layers = []
+    for ch in pattern:
+        if ch in "Kk":
+            kind, mix = "attention", NormedAttnSpec(heads, kv_heads, dim, dim, dim ** -0.5, row_norm=True, bias=True,
+                                                    key_values=True, temp_coef=temp[0], temp_every=temp[1])
+        elif ch in "Rr":
+            rd = rot_dim or dim
+            rot = RotarySpec(rot_dims or rd, 500000.0, half=True,
+                             **(dict(zip(("factor", "low", "high", "original"), scaling)) if scaling else {}))
+            kind, mix = "attention_2", NormedAttnSpec(rot_heads or heads, rot_kv_heads or kv_heads, rd, vdim or rd, rd ** -0.5,
+                                                      rot=rot, softcap=softcap, sink=True, gate=True)
+        else:
+            raise ValueError(f"pattern letter {ch!r}")
+        layers.append(BekedraLayer(kind, mix, ChosenSoftmaxSpec(experts, top, expert_ff) if ch.isupper() else None))
+    return BekedraConfig(name=name, vocab_size=vocab, hidden_size=width, layers=tuple(layers),
+                         loop=LoopSpec(*loop) if loop else None, embed_scale=embed_scale, **kw)
+
+
+TINY_BEKEDRA = bekedra_stack("tiny-bekedra", 512, 128, "RKR", heads=4, kv_heads=2, dim=32, experts=6, top=2, expert_ff=64,
+                             rot_dims=16, rot_heads=2, rot_kv_heads=1, rot_dim=48, loop=(1, 3, 2), embed_scale=4.0,
+                             scaling=(4.0, 1.0, 4.0, 256.0), softcap=20.0, temp=(0.2, 50), max_position=2048,
+                             bos_token_id=500, eos_token_ids=(501, 502))
+# layer shapes of a mid-size model (benchmarks; random weights)
+SMALL_BEKEDRA = bekedra_stack("small-bekedra", 32768, 2048, "RKKR", heads=16, kv_heads=4, dim=128, experts=16, top=4,
+                              expert_ff=1536, embed_scale=8.0, max_position=8192, bos_token_id=32000,
+                              eos_token_ids=(32001, 32002))
+
 LLAMA31_SCALING = {
     "rope_type": "llama3",
     "factor": 8.0,
@@ -1263,7 +1483,7 @@ _REGISTRY = {
     for c in (LLAMA3_8B, LLAMA31_8B, LLAMA3_70B, LLAMA31_70B, MIXTRAL_8X7B, TINY_LLAMA, TINY_MIXTRAL, SMALL_LLAMA,
               TINY_LLAMA_KV8, TINY_MIXTRAL_E8, TINY_BOZEVIK, SMALL_BOZEVIK, SMALL_BOZEVIK_MOE, TINY_LEMUNEX,
               SMALL_LEMUNEX, SMALL_LEMUNEX_MOE, TINY_KOMAZEN, SMALL_KOMAZEN, TINY_DALALIX, SMALL_DALALIX,
-              TINY_BELETAR, SMALL_BELETAR)
+              TINY_BELETAR, SMALL_BELETAR, TINY_BEKEDRA, SMALL_BEKEDRA)
 }
 _ALIASES = {
     "llama3": "llama3:8b",
@@ -1296,7 +1516,7 @@ def known_models() -> list[str]:
 
 def from_config_json(cfg: dict, name: str = "hf", shapes: dict | None = None):
     """The model configuration of a checkpoint directory's config.json: the design is chosen by its
-    ``architecture`` key (Bozevik, Lemunex, Komazen, Dalalix, Beletar), otherwise the HuggingFace Llama / Mixtral keys.  ``shapes``:
+    ``architecture`` key (Bozevik, Lemunex, Komazen, Dalalix, Beletar, Bekedra), otherwise the HuggingFace Llama / Mixtral keys.  ``shapes``:
     the checkpoint's tensor shapes, for designs that leave some sizes to them."""
     if cfg.get("architecture") == "Bozevik":
         return bozevik_from_config(cfg, name)
@@ -1308,6 +1528,8 @@ def from_config_json(cfg: dict, name: str = "hf", shapes: dict | None = None):
         return dalalix_from_config(cfg, name)
     if cfg.get("architecture") == "Beletar":
         return beletar_from_config(cfg, name, shapes)
+    if cfg.get("architecture") == "Bekedra":
+        return bekedra_from_config(cfg, name)
     return from_hf_config(cfg, name)
 
 

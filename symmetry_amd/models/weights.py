@@ -188,6 +188,8 @@ def random_weights(cfg: ModelConfig, shard: ShardSpec | None = None, device="cpu
         return dalalix_random_weights(cfg, shard, device, dtype, seed)
     if getattr(cfg, "family", "llama") == "beletar":
         return beletar_random_weights(cfg, shard, device, dtype, seed)
+    if getattr(cfg, "family", "llama") == "bekedra":
+        return bekedra_random_weights(cfg, shard, device, dtype, seed)
     shard.validate(cfg)
     shapes = full_shapes(cfg)
     tensors = {}
@@ -250,6 +252,8 @@ def load_hf_weights(path: str, cfg: ModelConfig, shard: ShardSpec | None = None,
         return load_dalalix_weights(path, cfg, shard, device, dtype)
     if getattr(cfg, "family", "llama") == "beletar":
         return load_beletar_weights(path, cfg, shard, device, dtype)
+    if getattr(cfg, "family", "llama") == "bekedra":
+        return load_bekedra_weights(path, cfg, shard, device, dtype)
     shard.validate(cfg)
     wmap = _hf_index(path)
     handles = {}
@@ -900,5 +904,100 @@ def save_beletar_checkpoint(weights: ModelWeights, path: str) -> None:
     os.makedirs(path, exist_ok=True)
     with open(os.path.join(path, "config.json"), "w") as f:
         json.dump(beletar_to_config(weights.cfg), f, indent=1)
+    save_file({k: v.detach().to(torch.bfloat16).contiguous().cpu() for k, v in weights.tensors.items()},
+              os.path.join(path, "model.safetensors"))
+
+
+# --------------------------------------------------------------------------------------------------
+# Bekedra checkpoints: tensors keep the checkpoint's names (embed, loop.step, l<i>.norm1, l<i>.mix.q, l<i>.mix.q.b,
+# l<i>.mix.q.norm, l<i>.mix.sink, l<i>.mlp.router, l<i>.mlp.e<j>.up, ..., final.norm); a layer that runs several times has
+# its tensors once.  models/bekedra.py fuses what its GEMMs read.
+# --------------------------------------------------------------------------------------------------
+def bekedra_shapes(cfg) -> dict:
+    """Tensor name -> shape."""
+    d = cfg.hidden_size
+    shapes = {"embed": (cfg.vocab_size, d), "final.norm": (d,)}
+    if cfg.loop:
+        shapes["loop.step"] = (cfg.loop.times, d)
+    for i, layer in enumerate(cfg.layers):
+        p, m, q = f"l{i}.", layer.mixer, f"l{i}.mix."
+        nq, nk = m.heads * m.dim, m.kv_heads * m.dim
+        shapes[p + "norm1"] = (d,)
+        shapes[q + "q"], shapes[q + "k"] = (nq, d), (nk, d)
+        if m.bias:
+            shapes[q + "q.b"], shapes[q + "k.b"] = (nq,), (nk,)
+        if not m.key_values:
+            shapes[q + "v"] = (m.kv_heads * m.vdim, d)
+        shapes[q + "q.norm"], shapes[q + "k.norm"] = ((nq,), (nk,)) if m.row_norm else ((m.dim,), (m.dim,))
+        if m.sink:
+            shapes[q + "sink"] = (m.heads,)
+        if m.gate:
+            shapes[q + "g"] = (m.heads * m.vdim, d)
+        shapes[q + "o"] = (d, m.heads * m.vdim)
+        if layer.mlp is not None:
+            f = layer.mlp
+            shapes[p + "mlp.router"], shapes[p + "mlp.router.b"] = (f.experts, d), (f.experts,)
+            for e in range(f.experts):
+                shapes[f"{p}mlp.e{e}.up"], shapes[f"{p}mlp.e{e}.down"] = (f.expert_ff, d), (d, f.expert_ff)
+    return shapes
+
+
+def bekedra_random_weights(cfg, shard: ShardSpec | None = None, device="cpu", dtype=torch.bfloat16,
+                           seed: int = 0) -> ModelWeights:
+    """Random init (benchmarks, tests): matrices N(0, (1.28 / sqrt(fan_in))^2); norm weights around one; biases, sinks and
+    the passes' vectors away from zero -- a dropped parameter shows."""
+    shard = shard or ShardSpec()
+    if shard.tp_size > 1 or shard.ep_size > 1:
+        raise NotImplementedError("Bekedra runs on one GPU per replica (its tensors are not sharded)")
+    tensors = {}
+    for name, shape in bekedra_shapes(cfg).items():
+        g = torch.Generator().manual_seed(_seed(seed, name))
+        leaf = name.rsplit(".", 1)[-1]
+        if leaf in ("norm", "norm1"):
+            t = 0.75 + 0.5 * torch.rand(shape, generator=g)
+        elif leaf == "b":
+            t = 0.3 * torch.randn(shape, generator=g)
+        elif leaf in ("sink", "step"):
+            t = torch.randn(shape, generator=g)
+        else:      # (the embedding table is the output head too: its rows are scaled like any matrix of this width)
+            tensors[name] = _randn(shape, _seed(seed, name), device, dtype, _std("head" if name == "embed" else name, shape))
+            continue
+        tensors[name] = t.to(dtype).to(device)
+    return ModelWeights(cfg, shard, tensors)
+
+
+def load_bekedra_weights(path: str, cfg, shard: ShardSpec | None = None, device="cpu",
+                         dtype=torch.bfloat16) -> ModelWeights:
+    """model.safetensors of a Bekedra checkpoint directory; every tensor the configuration implies must be there with the
+    implied shape, and no other.  Tensors stay in the file's precision (the model converts what it fuses)."""
+    from safetensors import safe_open
+
+    shard = shard or ShardSpec()
+    if shard.tp_size > 1 or shard.ep_size > 1:
+        raise NotImplementedError("Bekedra runs on one GPU per replica (its tensors are not sharded)")
+    shapes = bekedra_shapes(cfg)
+    tensors = {}
+    with safe_open(os.path.join(path, "model.safetensors"), framework="pt") as f:
+        names = set(f.keys())
+        missing, extra = sorted(set(shapes) - names), sorted(names - set(shapes))
+        if missing or extra:
+            raise ValueError(f"checkpoint does not fit its config: missing {missing[:4]}, unexpected {extra[:4]}")
+        for name, shape in shapes.items():
+            t = f.get_tensor(name)
+            if tuple(t.shape) != tuple(shape):
+                raise ValueError(f"{name}: shape {tuple(t.shape)}, the config implies {tuple(shape)}")
+            tensors[name] = t.to(device)
+    return ModelWeights(cfg, shard, tensors)
+
+
+def save_bekedra_checkpoint(weights: ModelWeights, path: str) -> None:
+    """config.json + model.safetensors (bf16) of a Bekedra model, in the form the loader reads."""
+    from safetensors.torch import save_file
+
+    from .config import bekedra_to_config
+
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(bekedra_to_config(weights.cfg), f, indent=1)
     save_file({k: v.detach().to(torch.bfloat16).contiguous().cpu() for k, v in weights.tensors.items()},
               os.path.join(path, "model.safetensors"))

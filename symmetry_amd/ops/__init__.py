@@ -633,6 +633,11 @@ def rope_pair_table(max_pos: int, dims: int, base: float, device=None) -> torch.
     return reference.rope_pair_table(max_pos, dims, base, device)
 
 
+def rope_table(max_pos: int, dims: int, base: float, scaling: dict | None = None) -> torch.Tensor:
+    """[max_pos, cos | sin] fp32 of the angles p * base^(-2 i / dims), with Llama-3.1 frequency scaling by wavelength."""
+    return reference.rope_table(max_pos, dims, base, scaling)
+
+
 def latent_prep(z, q_rank, kv_rank, rot, wq, wkv, eps, positions, slots, rope, cq, cache, half_dims=0):
     """z [T, q_rank (+ kv_rank + rot)] (a view: further columns may follow in its rows) -> cq = rms_norm(z[:, :q_rank]) *
     wq; with a kv part (kv_rank > 0) the token's cache row (slot >= 0) becomes [rms_norm(z kv part) * wkv | rotary(z rot
@@ -776,20 +781,22 @@ WINDOW_ATTN_IMPL = 0 if os.environ.get("SYMMETRY_WINDOW_ATTN", "auto") == "wave"
 
 
 def window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, window, scale, gate, out, tiles=None, cu_q=None,
-                impl=None, bias=None, keep_first=0, sink=None):
+                impl=None, bias=None, keep_first=0, sink=None, softcap=0.0, key_scale=None):
     """Softmax attention of q [T, H, dk] over the paged caches: row r sees positions max(0, p - window + 1) .. p of
     sequence row_seq[r] (p = positions[r]) and, with ``keep_first``, the sequence's first keep_first positions; query
-    head h reads key / value head h // (H / G); scores and weights fp32.  ``gate`` [T, H] (a view): head outputs are
-    multiplied by sigmoid(gate).  ``tiles`` / ``cu_q``: the packed prompt form (64-row query tiles), for the tiled
+    head h reads key / value head h // (H / G); scores and weights fp32.  ``gate`` [T, H] or [T, H dv] (a view): head outputs, or
+    their entries one by one, are multiplied by sigmoid(gate).  ``tiles`` / ``cu_q``: the packed prompt form (64-row query tiles), for the tiled
     kernel.  Returns the implementation used (0: one wave per (row, head), every shape; 1: tiled).  ``bias`` [2, H] fp32:
     the score of a key at distance n = p - j is lowered by bias[0, h] * ln(1 + bias[1, h] * n).  ``sink`` [H] fp32: the
-    softmax's denominator of head h also holds exp(sink[h]) (a logit without a key or a value, not scaled)."""
+    softmax's denominator of head h also holds exp(sink[h]) (a logit without a key or a value, not scaled or capped).
+    ``key_scale`` [NB, BS] fp32: the scores of a key are multiplied by its cache row's number; ``softcap`` c > 0: scores
+    become c tanh(s / c) (before the distance bias).  ``v_cache`` may be ``k_cache`` itself."""
     if _gpu(q):
         return _hyb().window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, int(window), float(scale), gate,
                                   out, tiles, cu_q, WINDOW_ATTN_IMPL if impl is None else int(impl), bias,
-                                  int(keep_first), sink)
+                                  int(keep_first), sink, float(softcap), key_scale)
     reference.window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, window, scale, gate, out, bias,
-                          keep_first, sink)
+                          keep_first, sink, softcap, key_scale)
     return 0
 
 
@@ -936,14 +943,15 @@ def post_rms_norm(x, alpha, delta, w, eps, conv_w=None, conv_state=None, prev_ro
         reference.conv_state_update(x, conv_state, None, prev_row, save_slot, runs)
 
 
-def qk_norm_cache(z, H, G, dk, dv, wq, wk, q_mult, eps, slots, q_out, k_cache, v_cache):
+def qk_norm_cache(z, H, G, dk, dv, wq, wk, q_mult, eps, slots, q_out, k_cache, v_cache, rope=None, positions=None):
     """z [T, H dk | G dk | G dv (| ...)] -> q_out [T, H, dk] = rms_norm per head (weight wq [dk], shared by the heads)
     times q_mult[h] (optional); the token's rows of the paged caches k [NB, BS, G, dk] = rms_norm per head (wk),
-    v [NB, BS, G, dv] (slot >= 0).  Statistics fp32."""
+    v [NB, BS, G, dv] (slot >= 0).  ``rope`` [max_pos, pairs, 2]: the normed queries and keys turn on their first
+    2 * pairs entries (half layout: entry i with entry i + pairs) at ``positions``.  Statistics and rotation fp32."""
     if _gpu(z):
         return _hyb().qk_norm_cache(z, int(H), int(G), int(dk), int(dv), wq, wk, q_mult, float(eps), slots, q_out,
-                                    k_cache, v_cache)
-    return reference.qk_norm_cache(z, H, G, dk, dv, wq, wk, q_mult, eps, slots, q_out, k_cache, v_cache)
+                                    k_cache, v_cache, rope, positions)
+    return reference.qk_norm_cache(z, H, G, dk, dv, wq, wk, q_mult, eps, slots, q_out, k_cache, v_cache, rope, positions)
 
 
 def gelu_tanh_mul(gate, up, out):
@@ -1085,3 +1093,42 @@ def delta_rule(channel, q, k, v, dz, dt_bias, A_log, bz, state, cu_q, prev_row, 
                                  out, tiles, ws, DELTA_IMPL if impl is None else int(impl))
     reference.delta_rule(channel, q, k, v, dz, dt_bias, A_log, bz, state, cu_q, prev_row, save_slot, runs, out)
     return 1
+
+
+# ---- attention whose values are its keys, routed squared-ReLU experts (csrc/kernels/hybrid_rows.hip, routed_ff.hip) ----
+def qk_row_norm_cache(z, bias, H, G, dk, wq, wk, eps, temp_coef, temp_every, positions, slots, q_out, kv_cache, key_scale):
+    """z [T, H dk | G dk (| ...)] + bias (fp32, optional), query and key each under one RMS norm over its whole projection
+    (weights wq [H dk], wk [G dk]).  The cache keeps the key as projected, kv_cache [NB, BS, G, dk] (its value as well), and
+    the norm's statistic key_scale [NB, BS] fp32 = 1 / rms (slot >= 0); the key weight goes into the query:
+    q_out [T, H, dk] = q / rms * wq * wk(group) * (1 + temp_coef ln(floor((p + 1) / temp_every) + 1)), so that
+    key_scale * (q_out . kv_cache row) is the score of the normed pair.  Statistics fp32."""
+    if _gpu(z):
+        return _hyb().qk_row_norm_cache(z, bias, int(H), int(G), int(dk), wq, wk, float(eps), float(temp_coef),
+                                        int(temp_every), positions, slots, q_out, kv_cache, key_scale)
+    return reference.qk_row_norm_cache(z, bias, H, G, dk, wq, wk, eps, temp_coef, temp_every, positions, slots, q_out,
+                                       kv_cache, key_scale)
+
+
+def route_topk(x, Wr, bias, k, ids, w, offsets, dst, src):
+    """Router: logits x @ Wr.T + bias (fp32; bias optional), the k largest (ties: the lowest index) -> ids [T k], w = softmax
+    over the chosen logits; and the routed rows' places in expert order: offsets [E + 1] segment bounds, dst [T k] place of
+    every (token, choice), src [T k] token of every place."""
+    if _gpu(x):
+        return _hyb().route_topk(x, Wr, bias, int(k), ids, w, offsets, dst, src)
+    return reference.route_topk(x, Wr, bias, k, ids, w, offsets, dst, src)
+
+
+def expert_linear(x, src, W, offsets, y, relu2=False):
+    """y[i] = W[e] x[src[i]] (src None: x[i]) for the places i of expert e's segment, W [E, N, K]; ``relu2``: relu(.)^2.
+    Segment bounds are read on the device (no host sync)."""
+    if _gpu(x):
+        return _hyb().expert_linear(x, src, W, offsets, y, bool(relu2))
+    return reference.expert_linear(x, src, W, offsets, y, relu2)
+
+
+def residual_routed_norm(x, a, y, dst, w, k, bias, wn=None, eps=0.0, out=None):
+    """x += a + sum_j w[t k + j] y[dst[t k + j]] + bias in fp32 (a, y, bias each optional); with ``out``: out = x / rms * wn,
+    the next layer's normalised input, from the same pass."""
+    if _gpu(x):
+        return _hyb().residual_routed_norm(x, a, y, dst, w, int(k), bias, wn, float(eps), out)
+    return reference.residual_routed_norm(x, a, y, dst, w, k, bias, wn, eps, out)

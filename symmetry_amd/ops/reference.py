@@ -802,7 +802,7 @@ def qkv_rope_cache(z, bias, H, G, dk, dv, positions, slots, rope, q_out, k_cache
 
 
 def window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, window, scale, gate, out, bias=None, keep_first=0,
-                sink=None) -> None:
+                sink=None, softcap=0.0, key_scale=None) -> None:
     T, H, dk = q.shape
     BS, G = k_cache.shape[1], k_cache.shape[2]
     rep = H // G
@@ -815,6 +815,10 @@ def window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, window, s
         V = v_cache[bt[idx // BS], idx % BS].float()
         qr = q[r].float().view(G, rep, dk)
         s = torch.einsum("grd,ngd->grn", qr, K) * scale
+        if key_scale is not None:
+            s = s * key_scale[bt[idx // BS], idx % BS].float()
+        if softcap > 0:
+            s = softcap * torch.tanh(s / softcap)
         if bias is not None:     # [2, H]: score -= bias[0, h] * ln(1 + bias[1, h] * distance)
             dist = (p - idx).float()
             s = s - (bias[0].float()[:, None] * torch.log1p(bias[1].float()[:, None] * dist[None, :])).view(G, rep, -1)
@@ -822,8 +826,8 @@ def window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, window, s
             s = torch.cat([s, sink.float().view(G, rep, 1)], -1)
             V = torch.cat([V, torch.zeros_like(V[:1])], 0)
         o = torch.einsum("grn,ngv->grv", torch.softmax(s, -1), V).reshape(H, -1)
-        if gate is not None:
-            o = o * torch.sigmoid(gate[r].float())[:, None]
+        if gate is not None:     # [T, H] or [T, H dv]
+            o = o * torch.sigmoid(gate[r].float()).view(H, -1)
         out[r] = o.to(out.dtype)
 
 
@@ -1001,15 +1005,19 @@ def post_rms_norm(x, alpha, delta, w, eps) -> None:
     x.copy_(_unit_rms(alpha * x + delta.float().view_as(x), eps) * w.float())
 
 
-def qk_norm_cache(z, H, G, dk, dv, wq, wk, q_mult, eps, slots, q_out, k_cache, v_cache) -> None:
+def qk_norm_cache(z, H, G, dk, dv, wq, wk, q_mult, eps, slots, q_out, k_cache, v_cache, rope=None, positions=None) -> None:
     T = z.shape[0]
     nq, nk, nv = H * dk, G * dk, G * dv
     zf = z[:, :nq + nk + nv].float()
     q = _unit_rms(zf[:, :nq].view(T, H, dk), eps) * wq.float()
+    k = _unit_rms(zf[:, nq:nq + nk].view(T, G, dk), eps) * wk.float()
+    if rope is not None:
+        cs = rope[positions[:T].long()][:, None]                  # [T, 1, pairs, 2]
+        q, k = _rot_half(q, cs, 2 * rope.shape[1]), _rot_half(k, cs, 2 * rope.shape[1])
     if q_mult is not None:
         q = q * q_mult.float()[None, :, None]
     q_out.copy_(q.to(q_out.dtype))
-    k = (_unit_rms(zf[:, nq:nq + nk].view(T, G, dk), eps) * wk.float()).to(k_cache.dtype)
+    k = k.to(k_cache.dtype)
     v = zf[:, nq + nk:].view(T, G, dv).to(v_cache.dtype)
     sl = slots[:T].long()
     keep = sl >= 0
@@ -1144,3 +1152,67 @@ def delta_rule(channel, q, k, v, dz, dt_bias, A_log, bz, state, cu_q, prev_row, 
         sv = int(save_slot[s1 - 1])
         if sv >= 0:
             state[sv] = S
+
+
+# ---- attention whose values are its keys, routed squared-ReLU experts beside the mixer (the Bekedra layers) ------------
+def qk_row_norm_cache(z, bias, H, G, dk, wq, wk, eps, temp_coef, temp_every, positions, slots, q_out, kv_cache,
+                      key_scale) -> None:
+    T, nq, nk = z.shape[0], H * dk, G * dk
+    zf = z[:, :nq + nk].float()
+    if bias is not None:
+        zf = zf + bias.float()
+    q = _unit_rms(zf[:, :nq], eps) * wq.float()
+    if temp_coef:
+        p = positions[:T].long()
+        q = q * (1.0 + temp_coef * torch.log((torch.div(p + 1, temp_every, rounding_mode="floor") + 1).float()))[:, None]
+    # the key norm's weight is a factor of the query, its statistic one number per key
+    q = q.view(T, G, H // G, dk) * wk.float().view(1, G, 1, dk)
+    q_out.copy_(q.reshape(T, H, dk).to(q_out.dtype))
+    k = zf[:, nq:]
+    sl = slots[:T].long()
+    keep = sl >= 0
+    kv_cache.view(-1, nk)[sl[keep]] = k[keep].to(kv_cache.dtype)
+    key_scale.view(-1)[sl[keep]] = torch.rsqrt((k * k).mean(-1) + eps)[keep]
+
+
+def route_topk(x, Wr, bias, k, ids, w, offsets, dst, src) -> None:
+    T, E = x.shape[0], Wr.shape[0]
+    z = x.float() @ Wr.float().t()
+    if bias is not None:
+        z = z + bias.float()
+    pick = torch.argsort(z, dim=-1, descending=True, stable=True)[:, :k]
+    ids[: T * k].copy_(pick.reshape(-1).int())
+    w[: T * k].copy_(torch.softmax(torch.gather(z, 1, pick), -1).reshape(-1))
+    flat = pick.reshape(-1)
+    counts = torch.bincount(flat, minlength=E)
+    offsets[0] = 0
+    offsets[1:E + 1] = torch.cumsum(counts, 0).int()
+    order = torch.argsort(flat, stable=True)
+    dst[order] = torch.arange(T * k, dtype=torch.int32)
+    src[: T * k].copy_((order // k).int())
+
+
+def expert_linear(x, src, W, offsets, y, relu2=False) -> None:
+    for e in range(W.shape[0]):
+        a, b = int(offsets[e]), int(offsets[e + 1])
+        if b <= a:
+            continue
+        rows = x[src[a:b].long()] if src is not None else x[a:b]
+        p = rows.float() @ W[e].float().t()
+        if relu2:
+            p = torch.relu(p) ** 2
+        y[a:b] = p.to(y.dtype)
+
+
+def residual_routed_norm(x, a, y, dst, w, k, bias, wn, eps, out) -> None:
+    s = torch.zeros_like(x)
+    if a is not None:
+        s = s + a.float().view_as(x)
+    if y is not None:
+        T = x.shape[0]
+        s = s + (w[: T * k].view(T, k, 1) * y.float()[dst[: T * k].long()].view(T, k, -1)).sum(1)
+    if bias is not None:
+        s = s + bias.float()
+    x.add_(s)
+    if out is not None:
+        out.copy_((_unit_rms(x, eps) * wn.float()).to(out.dtype))
