@@ -1,6 +1,6 @@
-// TORCH_LIBRARY registration of the kernels in hybrid_rows.hip, stream_rows.hip, window_attention.hip, decay_scan.hip and
-// delta_rule.hip, plus the expert-segment kernels of glu_moe.hip that the routed feed-forward shares (symmetry_amd/_C_hybrid.so, namespace
-// symmetry_amd_hybrid).
+// TORCH_LIBRARY registration of the kernels in hybrid_rows.hip, stream_rows.hip, norm_rows.hip, routed_ff.hip,
+// window_attention.hip, decay_scan.hip and delta_rule.hip, plus the expert-segment kernels of glu_moe.hip that the routed
+// feed-forward shares (symmetry_amd/_C_hybrid.so, namespace symmetry_amd_hybrid).
 //
 // Out-parameter style like the other kernel libraries: the caller pre-allocates, nothing is allocated here, every
 // launch goes to torch's current HIP stream (hipGraph-capturable), and every shape / dtype / range the kernels and
@@ -184,7 +184,7 @@ void qkv_rope_cache(const Tensor& z, const OptTensor& bias, int64_t H, int64_t G
 int64_t window_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache, const Tensor& block_tables,
                     const Tensor& row_seq, const Tensor& positions, int64_t window, double scale, const OptTensor& gate,
                     Tensor& out, const OptTensor& tiles, const OptTensor& cu_q, int64_t impl, const OptTensor& bias,
-                    int64_t keep_first, const OptTensor& sink) {
+                    int64_t keep_first, const OptTensor& sink, double softcap, const OptTensor& key_scale) {
   const int f32 = act(q, "q");
   same_act(k_cache, f32, "k_cache");
   same_act(v_cache, f32, "v_cache");
@@ -203,7 +203,10 @@ int64_t window_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cach
                   a.T <= 65535 && k_cache.size(0) * k_cache.size(1) < (1LL << 31),
               "window_attn: shapes");
   if (gate.has_value()) {
-    a.ldg = view2(*gate, f32, a.T, a.H, "gate");
+    TORCH_CHECK(gate->dim() == 2 && (gate->size(1) == a.H || gate->size(1) == (int64_t)a.H * a.dv),
+                "window_attn: gate [T, H] or [T, H dv]");
+    a.gate_cols = a.dv > 1 && gate->size(1) != a.H;
+    a.ldg = view2(*gate, f32, a.T, gate->size(1), "gate");
     a.gate = gate->data_ptr();
   }
   if (bias.has_value()) {
@@ -216,6 +219,12 @@ int64_t window_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cach
     TORCH_CHECK(sink->numel() == a.H, "window_attn: sink [H]");
     a.sink = ptr<float>(*sink);
   }
+  if (key_scale.has_value()) {
+    dtype(*key_scale, at::kFloat, "key_scale");
+    TORCH_CHECK(key_scale->numel() == k_cache.size(0) * k_cache.size(1), "window_attn: key_scale [blocks, BS]");
+    a.key_scale = ptr<float>(*key_scale);
+  }
+  a.softcap = (float)softcap;
   TORCH_CHECK(keep_first >= 0 && keep_first < (1LL << 30), "window_attn: keep_first");
   a.keep_first = (int)keep_first;
   if (tiles.has_value() && cu_q.has_value()) {
@@ -544,7 +553,7 @@ void post_rms_norm(Tensor& x, double alpha, const Tensor& delta, const Tensor& w
 
 void qk_norm_cache(const Tensor& z, int64_t H, int64_t G, int64_t dk, int64_t dv, const Tensor& wq, const Tensor& wk,
                    const OptTensor& q_mult, double eps, const Tensor& slots, Tensor& q_out, Tensor& k_cache,
-                   Tensor& v_cache) {
+                   Tensor& v_cache, const OptTensor& rope, const OptTensor& positions) {
   const int f32 = act(z, "z", false);
   TORCH_CHECK(z.dim() == 2, "qk_norm_cache: z [T, n]");
   const int64_t T = z.size(0), n = H * dk + G * dk + G * dv;
@@ -566,6 +575,14 @@ void qk_norm_cache(const Tensor& z, int64_t H, int64_t G, int64_t dk, int64_t dv
     TORCH_CHECK(q_mult->numel() == H, "qk_norm_cache: q_mult [H]");
     a.q_mult = ptr<float>(*q_mult);
   }
+  if (rope.has_value()) {
+    dtype(*rope, at::kFloat, "rope");
+    TORCH_CHECK(positions.has_value(), "qk_norm_cache: rope without positions");
+    dtype(*positions, at::kInt, "positions");
+    TORCH_CHECK(rope->dim() == 3 && rope->size(2) == 2 && 2 * rope->size(1) <= dk && positions->numel() >= T,
+                "qk_norm_cache: rope [max_pos, pairs, 2]");
+    a.rope = ptr<float>(*rope), a.positions = ptr<int>(*positions), a.pairs = (int)rope->size(1);
+  }
   a.z = z.data_ptr();
   a.H = (int)H, a.G = (int)G, a.dk = (int)dk, a.dv = (int)dv;
   a.wq = ptr<float>(wq), a.wk = ptr<float>(wk);
@@ -575,6 +592,125 @@ void qk_norm_cache(const Tensor& z, int64_t H, int64_t G, int64_t dk, int64_t dv
   a.k_cache = k_cache.data_ptr();
   a.v_cache = v_cache.data_ptr();
   launch_qk_norm_cache(a, (int)T, f32, cur_stream(z));
+}
+
+void qk_row_norm_cache(const Tensor& z, const OptTensor& bias, int64_t H, int64_t G, int64_t dk, const Tensor& wq,
+                       const Tensor& wk, double eps, double coef, int64_t every, const Tensor& positions,
+                       const Tensor& slots, Tensor& q_out, Tensor& kv_cache, Tensor& key_scale) {
+  const int f32 = act(z, "z", false);
+  TORCH_CHECK(z.dim() == 2, "qk_row_norm_cache: z [T, n]");
+  const int64_t T = z.size(0), n = H * dk + G * dk;
+  QkRowNormArgs a{};
+  a.ldz = view2(z, f32, T, z.size(1), "z");
+  same_act(q_out, f32, "q_out");
+  same_act(kv_cache, f32, "kv_cache");
+  dtype(wq, at::kFloat, "wq");
+  dtype(wk, at::kFloat, "wk");
+  dtype(key_scale, at::kFloat, "key_scale");
+  dtype(positions, at::kInt, "positions");
+  dtype(slots, at::kInt, "slots");
+  TORCH_CHECK(z.size(1) >= n && G > 0 && H % G == 0 && wq.numel() == H * dk && wk.numel() == G * dk &&
+                  q_out.numel() == T * H * dk && kv_cache.dim() == 4 && kv_cache.size(2) == G && kv_cache.size(3) == dk &&
+                  key_scale.numel() == kv_cache.size(0) * kv_cache.size(1) && positions.numel() >= T && slots.numel() >= T &&
+                  every >= 1, "qk_row_norm_cache: shapes");
+  if (bias.has_value()) {
+    dtype(*bias, at::kFloat, "bias");
+    TORCH_CHECK(bias->numel() == n, "qk_row_norm_cache: bias [H dk + G dk]");
+    a.bias = ptr<float>(*bias);
+  }
+  a.z = z.data_ptr();
+  a.H = (int)H, a.G = (int)G, a.dk = (int)dk;
+  a.wq = ptr<float>(wq), a.wk = ptr<float>(wk);
+  a.eps = (float)eps, a.coef = (float)coef, a.every = (int)every;
+  a.positions = ptr<int>(positions), a.slots = ptr<int>(slots);
+  a.q_out = q_out.data_ptr(), a.kv_cache = kv_cache.data_ptr(), a.key_scale = ptr<float>(key_scale);
+  launch_qk_row_norm_cache(a, (int)T, f32, cur_stream(z));
+}
+
+void route_topk(const Tensor& x, const Tensor& Wr, const OptTensor& bias, int64_t k, Tensor& ids, Tensor& w, Tensor& offsets,
+                Tensor& dst, Tensor& src) {
+  const int f32 = act(x, "x");
+  same_act(Wr, f32, "Wr");
+  dtype(w, at::kFloat, "w");
+  for (const Tensor* t : {&ids, &offsets, &dst, &src}) dtype(*t, at::kInt, "ids / offsets / dst / src");
+  TORCH_CHECK(x.dim() == 2 && Wr.dim() == 2 && Wr.size(1) == x.size(1), "route_topk: x [T, d], Wr [E, d]");
+  RouteArgs a{};
+  const int64_t T = x.size(0), E = Wr.size(0);
+  TORCH_CHECK(k >= 1 && k <= E && E <= 1024 && T * k < (1LL << 30) && ids.numel() >= T * k && w.numel() >= T * k &&
+                  dst.numel() >= T * k && src.numel() >= T * k && offsets.numel() >= E + 1, "route_topk: shapes");
+  if (bias.has_value()) {
+    dtype(*bias, at::kFloat, "bias");
+    TORCH_CHECK(bias->numel() == E, "route_topk: bias [E]");
+    a.bias = ptr<float>(*bias);
+  }
+  a.x = x.data_ptr(), a.Wr = Wr.data_ptr();
+  a.T = (int)T, a.d = (int)x.size(1), a.E = (int)E, a.k = (int)k;
+  a.ids = ptr<int>(ids), a.w = ptr<float>(w), a.offsets = ptr<int>(offsets), a.dst = ptr<int>(dst), a.src = ptr<int>(src);
+  launch_route_topk(a, f32, cur_stream(x));
+}
+
+int64_t expert_linear(const Tensor& x, const OptTensor& src, const Tensor& W, const Tensor& offsets, Tensor& y, bool relu2,
+                      int64_t impl) {
+  const int f32 = act(x, "x");
+  same_act(W, f32, "W");
+  same_act(y, f32, "y");
+  dtype(offsets, at::kInt, "offsets");
+  TORCH_CHECK(x.dim() == 2 && W.dim() == 3 && y.dim() == 2, "expert_linear: x [T, K], W [E, N, K], y [R, N]");
+  ExpertArgs a{};
+  const int64_t R = y.size(0), E = W.size(0);
+  TORCH_CHECK(W.size(2) == x.size(1) && y.size(1) == W.size(1) && offsets.numel() >= E + 1 && (R + 63) / 64 + E <= 65535,
+              "expert_linear: shapes");
+  if (src.has_value()) {
+    dtype(*src, at::kInt, "src");
+    TORCH_CHECK(src->numel() >= R, "expert_linear: src [R]");
+    a.src = ptr<int>(*src);
+  } else {
+    TORCH_CHECK(x.size(0) >= R, "expert_linear: fewer rows of x than places");
+  }
+  a.x = x.data_ptr(), a.W = W.data_ptr(), a.offsets = ptr<int>(offsets), a.y = y.data_ptr();
+  a.R = (int)R, a.E = (int)E, a.N = (int)W.size(1), a.K = (int)W.size(2), a.relu2 = relu2;
+  return launch_expert_linear(a, f32, (int)impl, cur_stream(x));
+}
+
+void residual_routed_norm(Tensor& x, const OptTensor& a_, const OptTensor& y, const OptTensor& dst, const OptTensor& w,
+                          int64_t k, const OptTensor& bias, const OptTensor& wn, double eps, OptTensor out) {
+  dtype(x, at::kFloat, "x");
+  TORCH_CHECK(x.dim() == 2, "residual_routed_norm: x [T, d]");
+  RoutedSumArgs a{};
+  const int64_t T = x.size(0), d = x.size(1);
+  int f32 = -1;      // the activation dtype, from whichever activation there is
+  const auto same = [&](const Tensor& t, const char* name) {
+    const int v = act(t, name);
+    TORCH_CHECK(f32 < 0 || f32 == v, name, ": activation dtypes differ");
+    f32 = v;
+  };
+  if (a_.has_value()) {
+    same(*a_, "a");
+    TORCH_CHECK(a_->numel() == T * d, "residual_routed_norm: a [T, d]");
+    a.a = a_->data_ptr();
+  }
+  if (y.has_value()) {
+    same(*y, "y");
+    TORCH_CHECK(dst.has_value() && w.has_value() && k >= 1 && k <= 64, "residual_routed_norm: y without dst / w (k at most 64)");
+    dtype(*dst, at::kInt, "dst");
+    dtype(*w, at::kFloat, "w");
+    TORCH_CHECK(y->dim() == 2 && y->size(1) == d && y->size(0) >= T * k && dst->numel() >= T * k && w->numel() >= T * k,
+                "residual_routed_norm: y [T k, d], dst / w [T k]");
+    a.y = y->data_ptr(), a.dst = ptr<int>(*dst), a.w = ptr<float>(*w), a.k = (int)k;
+  }
+  if (bias.has_value()) {
+    dtype(*bias, at::kFloat, "bias");
+    TORCH_CHECK(bias->numel() == d, "residual_routed_norm: bias [d]");
+    a.bias = ptr<float>(*bias);
+  }
+  if (out.has_value()) {
+    same(*out, "out");
+    TORCH_CHECK(wn.has_value() && out->numel() == T * d && wn->numel() == d, "residual_routed_norm: out [T, d], wn [d]");
+    dtype(*wn, at::kFloat, "wn");
+    a.out = out->data_ptr(), a.wn = ptr<float>(*wn);
+  }
+  a.x = ptr<float>(x), a.eps = (float)eps, a.T = (int)T, a.d = (int)d;
+  launch_residual_routed_norm(a, f32 > 0, cur_stream(x));
 }
 
 void gelu_tanh_mul(const Tensor& gate, const Tensor& up, Tensor& out) {
@@ -958,7 +1094,7 @@ TORCH_LIBRARY(symmetry_amd_hybrid, m) {
   m.def(
       "window_attn(Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor row_seq, Tensor positions, "
       "int window, float scale, Tensor? gate, Tensor(a!) out, Tensor? tiles, Tensor? cu_q, int impl, Tensor? bias, "
-      "int keep_first, Tensor? sink) -> int",
+      "int keep_first, Tensor? sink, float softcap=0., Tensor? key_scale=None) -> int",
       &window_attn);
   m.def(
       "decay_scan(int mode, Tensor q, Tensor k, Tensor v, Tensor dz, Tensor dbias, Tensor? rate, float tau, Tensor? skip, "
@@ -1002,8 +1138,23 @@ TORCH_LIBRARY(symmetry_amd_hybrid, m) {
       &post_rms_norm);
   m.def(
       "qk_norm_cache(Tensor z, int H, int G, int dk, int dv, Tensor wq, Tensor wk, Tensor? q_mult, float eps, Tensor slots, "
-      "Tensor(a!) q_out, Tensor(b!) k_cache, Tensor(c!) v_cache) -> ()",
+      "Tensor(a!) q_out, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor? rope=None, Tensor? positions=None) -> ()",
       &qk_norm_cache);
+  m.def(
+      "qk_row_norm_cache(Tensor z, Tensor? bias, int H, int G, int dk, Tensor wq, Tensor wk, float eps, float coef, int every, "
+      "Tensor positions, Tensor slots, Tensor(a!) q_out, Tensor(b!) kv_cache, Tensor(c!) key_scale) -> ()",
+      &qk_row_norm_cache);
+  m.def(
+      "route_topk(Tensor x, Tensor Wr, Tensor? bias, int k, Tensor(a!) ids, Tensor(b!) w, Tensor(c!) offsets, Tensor(d!) dst, "
+      "Tensor(e!) src) -> ()",
+      &route_topk);
+  m.def(
+      "expert_linear(Tensor x, Tensor? src, Tensor W, Tensor offsets, Tensor(a!) y, bool relu2, int impl=-1) -> int",
+      &expert_linear);
+  m.def(
+      "residual_routed_norm(Tensor(a!) x, Tensor? a, Tensor? y, Tensor? dst, Tensor? w, int k, Tensor? bias, Tensor? wn, "
+      "float eps, Tensor(b!)? out) -> ()",
+      &residual_routed_norm);
   m.def("gelu_tanh_mul(Tensor gate, Tensor up, Tensor(a!) out) -> ()", &gelu_tanh_mul);
   m.def("sigmoid_mul(Tensor a, Tensor gate, Tensor(a!) out) -> ()", &sigmoid_mul);
   m.def(

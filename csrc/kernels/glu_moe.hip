@@ -7,7 +7,8 @@
 //                    the expert's INPUT; the clamps make the expert non-linear in it, so it cannot move to the output)
 //   grouped_linear   y = xs @ W[e]^T over the expert segments, bounds read from device memory (no host sync);
 //                    64 x 64 tiles through LDS with fp32 accumulation, any N / K -- the all-shapes, both-dtypes
-//                    grouped GEMM (bf16 shapes that tile for the MFMA grouped kernels run on those instead)
+//                    grouped GEMM (bf16 shapes that tile for the MFMA grouped kernels run on those instead);
+//                   optionally with gathered rows (src) and a squared-ReLU epilogue
 //   gather_sum       per token: the sum of its experts' output rows (+ the shared expert's), fp32
 #include "common.h"
 #include "latent_launchers.h"
@@ -159,7 +160,7 @@ constexpr int BM = 64, BN = 64, BK = 16;
 template <typename T>
 __global__ __launch_bounds__(NT) void grouped_linear_kernel(const T* __restrict__ xs, const T* __restrict__ W,
                                                             const int* __restrict__ offsets, int E, int N, int K,
-                                                            T* __restrict__ y) {
+                                                            T* __restrict__ y, const int* __restrict__ src, int relu2) {
   __shared__ float As[BK][BM + 4];
   __shared__ float Bs[BK][BN + 4];
   int slot = blockIdx.y, e = 0, r0 = 0, r1 = 0;
@@ -182,7 +183,7 @@ __global__ __launch_bounds__(NT) void grouped_linear_kernel(const T* __restrict_
     for (int i = threadIdx.x; i < BM * BK; i += NT) {
       const int m = i / BK, kk = i - m * BK;
       const int r = r0 + m, c = k0 + kk;
-      As[kk][m] = (r < r1 && c < K) ? (float)xs[(long long)r * K + c] : 0.f;
+      As[kk][m] = (r < r1 && c < K) ? (float)xs[(long long)(src ? src[r] : r) * K + c] : 0.f;
     }
     for (int i = threadIdx.x; i < BN * BK; i += NT) {
       const int n = i / BK, kk = i - n * BK;
@@ -209,7 +210,9 @@ __global__ __launch_bounds__(NT) void grouped_linear_kernel(const T* __restrict_
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
-      if (n < N) y[(long long)r * N + n] = (T)acc[i][j];
+      float v = acc[i][j];
+      if (relu2) v = fmaxf(v, 0.f) * fmaxf(v, 0.f);
+      if (n < N) y[(long long)r * N + n] = (T)v;
     }
   }
 }
@@ -267,11 +270,13 @@ void launch_scatter_scaled(const void* x, const int* ids, const float* w, int k,
 }
 
 void launch_grouped_linear(const void* xs, const void* W, const int* offsets, int E, int R, int N, int K, void* y,
-                           int f32, hipStream_t s) {
+                           int f32, hipStream_t s, const int* src, int relu2) {
   if (R <= 0) return;
   dim3 grid((N + BN - 1) / BN, (R + BM - 1) / BM + E);
-  if (f32) grouped_linear_kernel<float><<<grid, NT, 0, s>>>((const float*)xs, (const float*)W, offsets, E, N, K, (float*)y);
-  else grouped_linear_kernel<bf16><<<grid, NT, 0, s>>>((const bf16*)xs, (const bf16*)W, offsets, E, N, K, (bf16*)y);
+  if (f32) grouped_linear_kernel<float><<<grid, NT, 0, s>>>((const float*)xs, (const float*)W, offsets, E, N, K, (float*)y,
+                                                           src, relu2);
+  else grouped_linear_kernel<bf16><<<grid, NT, 0, s>>>((const bf16*)xs, (const bf16*)W, offsets, E, N, K, (bf16*)y,
+                                                    src, relu2);
 }
 
 void launch_gather_sum(const void* y, const int* dst, int k, const void* extra, float* out, int T, int d, int f32,

@@ -1,5 +1,5 @@
-// Host-side launch entry points of the kernels in hybrid_rows.hip, stream_rows.hip, window_attention.hip, decay_scan.hip
-// and delta_rule.hip: the
+// Host-side launch entry points of the kernels in hybrid_rows.hip, stream_rows.hip, norm_rows.hip,
+// routed_ff.hip, window_attention.hip, decay_scan.hip and delta_rule.hip: the
 // mechanisms of models that put windowed softmax attention beside linear recurrences with decaying state, use
 // state-space layers with a carried convolution, and add mixer and feed-forward to the stream from one norm.
 //
@@ -103,7 +103,8 @@ struct NormConvArgs {
 void launch_post_rms_norm(float* x, float alpha, const void* delta, const float* w, float eps, int T, int d,
                           const NormConvArgs& cv, int f32, hipStream_t s);
 // z[t] = q (H dk) | k (G dk) | v (G dv); q_out [T][H][dk] = q / rms_head * wq * q_mult[h]; cache rows `slot` (>= 0):
-// k_cache [rows][G][dk] = k / rms_head * wk, v_cache [rows][G][dv] = v
+// k_cache [rows][G][dk] = k / rms_head * wk, v_cache [rows][G][dv] = v.  rope [max_pos][pairs][2] (optional): normed q and k
+// turn on their first 2 pairs entries (entry i with entry i + pairs)
 struct QkNormArgs {
   const void* z; long long ldz;
   int H, G, dk, dv;
@@ -111,6 +112,9 @@ struct QkNormArgs {
   const float* wk;      // [dk]
   const float* q_mult;  // [H] or null
   float eps;
+  const float* rope;
+  const int* positions;
+  int pairs;
   const int* slots;
   void* q_out;
   void* k_cache;
@@ -124,6 +128,68 @@ void launch_gelu_tanh_mul(const void* gate, long long ldg, const void* up, long 
 void launch_sigmoid_mul(const void* a, long long lda, const void* gate, long long ldg, void* out, int R, int F, int f32,
                         hipStream_t s);
 
+// ---- norm_rows.hip --------------------------------------------------------------------------------------
+// z[t] = q (H dk) | k (G dk), + bias (optional); q_out [T][H][dk] = q / rms(all of q) * wq * wk(head's group) * (1 + coef
+// ln(floor((p + 1) / every) + 1)); cache rows `slot` (>= 0): kv_cache [rows][G][dk] = k, key_scale [rows] = 1 / rms(all of k)
+struct QkRowNormArgs {
+  const void* z; long long ldz;
+  const float* bias;    // [H dk + G dk] or null
+  int H, G, dk;
+  const float* wq;      // [H dk]
+  const float* wk;      // [G dk]
+  float eps, coef;
+  int every;
+  const int* positions;
+  const int* slots;
+  void* q_out;
+  void* kv_cache;
+  float* key_scale;
+};
+void launch_qk_row_norm_cache(const QkRowNormArgs& a, int T, int f32, hipStream_t s);
+// x += a + sum_j w[t k + j] y[dst[t k + j]] + bias (a, y, bias each optional; a and y in the activation dtype);
+// out (optional, activation dtype) = x_new / rms * wn
+struct RoutedSumArgs {
+  float* x;
+  const void* a;
+  const void* y;
+  const int* dst;
+  const float* w;
+  int k;
+  const float* bias;    // [d]
+  const float* wn;      // [d]
+  float eps;
+  void* out;
+  int T, d;
+};
+void launch_residual_routed_norm(const RoutedSumArgs& a, int f32, hipStream_t s);
+
+// ---- routed_ff.hip --------------------------------------------------------------------------------------
+// logits = x . Wr[e] + bias (fp32); the k largest (ties: lowest index) -> ids, w = softmax over them; the routed rows in expert
+// order: offsets [E + 1], dst [T k] place of a choice, src [T k] token of a place
+struct RouteArgs {
+  const void* x;        // [T][d]
+  const void* Wr;       // [E][d]
+  const float* bias;    // [E] or null
+  int T, d, E, k;
+  int* ids;             // [T k]
+  float* w;             // [T k]
+  int* offsets;
+  int* dst;
+  int* src;
+};
+void launch_route_topk(const RouteArgs& a, int f32, hipStream_t s);
+// y[i] = W[e] x[src ? src[i] : i] (relu2: relu(.)^2) for the places i of expert e's segment, W [E][N][K], y [R][N]
+struct ExpertArgs {
+  const void* x;
+  const int* src;
+  const void* W;
+  const int* offsets;
+  void* y;
+  int R, E, N, K, relu2;
+};
+// impl -1: by shape; 0 all shapes, 1 weight stream, 2 / 3 tiles.  Returns the form used.
+int launch_expert_linear(const ExpertArgs& a, int f32, int impl, hipStream_t s);
+
 // ---- window_attention.hip ------------------------------------------------------------------------------
 struct WindowAttnArgs {
   const void* q;        // [T][H][dk]
@@ -132,8 +198,11 @@ struct WindowAttnArgs {
   const int* block_tables;  // [seqs][max_blocks]
   const int* row_seq;   // [T]
   const int* positions; // [T]: row sees positions max(0, p - window + 1) .. p
-  const void* gate;     // [T][H] (row stride ldg) or null: output times sigmoid(gate)
+  const void* gate;     // [T][H], or [T][H dv] with gate_cols (row stride ldg), or null: output times sigmoid(gate)
   long long ldg;
+  int gate_cols;        // 1: a gate per output column instead of per head
+  const float* key_scale;   // [blocks][BS] or null: factor of the scores of the key in that cache row
+  float softcap;        // > 0: scores through softcap tanh(s / softcap)
   const float* bias;    // [2][H] or null: score of a key at distance n lowered by bias[0][h] * ln(1 + bias[1][h] * n)
   const float* sink;    // [H] or null: the softmax's denominator also holds exp(sink[h])
   void* out;            // [T][H][dv]

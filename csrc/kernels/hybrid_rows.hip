@@ -14,7 +14,8 @@
 //   embed_scale         x = table[token] * scale                            (fp32 stream)
 //   residual_conv       sublayer input x + causal per-channel convolution of the fp32 stream, carried taps fp32
 //   post_rms_norm       norm after the sum: x = rms_norm(alpha x + delta) * w, in place on the fp32 stream
-//   qk_norm_cache       per-head RMS norm of queries (times a per-head factor) and keys, paged key / value cache write
+//   qk_norm_cache       per-head RMS norm of queries (times a per-head factor) and keys, optional half-layout rotary, paged
+//                       key / value cache write
 //   gelu_tanh_mul, sigmoid_mul   gated activations on column ranges of a fused projection
 //
 // One workgroup per row unless noted; columns strided over the threads (coalesced), any width.  All statistics,
@@ -552,13 +553,78 @@ __global__ __launch_bounds__(NT) void qk_norm_cache_kernel(QkNormArgs a) {
     } else if (slot >= 0) {
       dst = reinterpret_cast<T*>(a.k_cache) + ((long long)slot * a.G + (head - a.H)) * a.dk;
     }
-    if (dst)
-      for (int e = lane; e < a.dk; e += 64) dst[e] = (T)((float)src[e] * w[e] * r);
+    if (dst) {
+      const float* cs = a.rope ? a.rope + (long long)a.positions[row] * 2 * a.pairs : nullptr;   // [pairs][2]
+      for (int e = lane; e < a.dk; e += 64) {
+        float v = (float)src[e] * w[e] * r;
+        if (e < 2 * a.pairs) {                           // entry e turns with entry e +- pairs
+          const bool lo = e < a.pairs;
+          const int o = lo ? e + a.pairs : e - a.pairs, pi = lo ? e : o;
+          const float u = (float)src[o] * w[o] * r;
+          v = lo ? v * cs[2 * pi] - u * cs[2 * pi + 1] : v * cs[2 * pi] + u * cs[2 * pi + 1];
+        }
+        dst[e] = (T)v;
+      }
+    }
   }
   if (slot >= 0) {
     T* vc = reinterpret_cast<T*>(a.v_cache) + (long long)slot * nv;
     for (int i = blockIdx.y * NT + threadIdx.x; i < nv; i += gridDim.y * NT) vc[i] = z[nq + nk + i];
   }
+}
+
+// The same for bf16 and sizes in multiples of 8: LPH neighbouring lanes per head, 16-byte accesses; grid (T, ceil((H + 2 G) /
+// (NT / LPH))), value heads after the key heads.
+template <int LPH>
+__global__ __launch_bounds__(NT) void qk_norm_cache_vec_kernel(QkNormArgs a) {
+  const int row = blockIdx.x, head = blockIdx.y * (NT / LPH) + threadIdx.x / LPH, e = 8 * (threadIdx.x % LPH);
+  if (head >= a.H + 2 * a.G) return;                     // (whole groups of LPH lanes)
+  const int slot = a.slots[row];
+  const bf16* z = reinterpret_cast<const bf16*>(a.z) + (long long)row * a.ldz;
+  if (head >= a.H + a.G) {
+    const int g = head - a.H - a.G;
+    if (slot >= 0 && e < a.dv)
+      *reinterpret_cast<uint4*>(reinterpret_cast<bf16*>(a.v_cache) + ((long long)slot * a.G + g) * a.dv + e) =
+          *reinterpret_cast<const uint4*>(z + (long long)(a.H + a.G) * a.dk + (long long)g * a.dv + e);
+    return;
+  }
+  const bool isq = head < a.H, in = e < a.dk;
+  const bf16* src = z + (long long)head * a.dk;
+  float v[8], sq = 0.f;
+  if (in) {
+    load8(src + e, v);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) sq += v[i] * v[i];
+  }
+#pragma unroll
+  for (int o = LPH / 2; o > 0; o >>= 1) sq += __shfl_xor(sq, o, 64);
+  const float r = 1.f / sqrtf(sq / (float)a.dk + a.eps);
+  if (!in || (!isq && slot < 0)) return;
+  float w[8];
+  const float* wn = isq ? a.wq : a.wk;
+  load8f(wn + e, w);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] *= w[i] * r;
+  if (e < 2 * a.pairs) {                                 // the 8 entries turn with the 8 entries +- pairs
+    const bool lo = e < a.pairs;
+    const int o = lo ? e + a.pairs : e - a.pairs, pi = lo ? e : o;
+    const float* cs = a.rope + ((long long)a.positions[row] * a.pairs + pi) * 2;
+    float u[8];
+    load8(src + o, u);
+    load8f(wn + o, w);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const float2 t = *reinterpret_cast<const float2*>(cs + 2 * i);
+      const float uu = u[i] * w[i] * r;
+      v[i] = lo ? v[i] * t.x - uu * t.y : v[i] * t.x + uu * t.y;
+    }
+  }
+  const float qm = isq && a.q_mult ? a.q_mult[head] : 1.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] *= qm;
+  bf16* dst = isq ? reinterpret_cast<bf16*>(a.q_out) + ((long long)row * a.H + head) * a.dk
+                  : reinterpret_cast<bf16*>(a.k_cache) + ((long long)slot * a.G + (head - a.H)) * a.dk;
+  store8(dst + e, v);
 }
 
 template <typename T>
@@ -786,8 +852,28 @@ void launch_post_rms_norm(float* x, float alpha, const void* delta, const float*
   }
 }
 
+// lanes per head of the vectorised form (8 entries each), or 0 where the shapes do not allow it
+static int qk_vec_lanes(const QkNormArgs& a, int f32) {
+  const auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const int m = a.dk > a.dv ? a.dk : a.dv;
+  if (f32 || a.dk % 8 || a.dv % 8 || a.pairs % 8 || a.ldz % 8 || m > 512 || !al(a.z) || !al(a.wq) || !al(a.wk) ||
+      !al(a.q_out) || !al(a.k_cache) || !al(a.v_cache) || (a.rope && !al(a.rope)))
+    return 0;
+  return m <= 64 ? 8 : (m <= 128 ? 16 : (m <= 256 ? 32 : 64));
+}
+
 void launch_qk_norm_cache(const QkNormArgs& a, int T_, int f32, hipStream_t s) {
   if (T_ <= 0) return;
+  const int lph = qk_vec_lanes(a, f32);
+  if (lph) {
+    const int per = NT / lph;      // heads of q, k and v per workgroup
+    dim3 grid(T_, (a.H + 2 * a.G + per - 1) / per);
+    if (lph == 8) qk_norm_cache_vec_kernel<8><<<grid, NT, 0, s>>>(a);
+    else if (lph == 16) qk_norm_cache_vec_kernel<16><<<grid, NT, 0, s>>>(a);
+    else if (lph == 32) qk_norm_cache_vec_kernel<32><<<grid, NT, 0, s>>>(a);
+    else qk_norm_cache_vec_kernel<64><<<grid, NT, 0, s>>>(a);
+    return;
+  }
   dim3 grid(T_, (a.H + a.G + NT / 64 - 1) / (NT / 64));
   DISPATCH_T(f32, qk_norm_cache_kernel<T><<<grid, NT, 0, s>>>(a);)
 }

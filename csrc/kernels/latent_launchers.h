@@ -84,9 +84,9 @@ void launch_expert_offsets(const int* ids, int R, int E, int* offsets, int* curs
 // xs[dst[a]] = w[a] * x[a / k] with dst[a] = offsets[ids[a]] + (arrival order within the expert)
 void launch_scatter_scaled(const void* x, const int* ids, const float* w, int k, int R, int d, const int* offsets,
                            int* cursor, void* xs, int* dst, int f32, hipStream_t s);
-// y[r] = xs[r] @ W[e]^T for the rows r of expert e's segment (W [E][N][K])
+// y[r] = xs[src ? src[r] : r] @ W[e]^T (relu2: relu(.)^2) for the rows r of expert e's segment (W [E][N][K])
 void launch_grouped_linear(const void* xs, const void* W, const int* offsets, int E, int R, int N, int K, void* y,
-                           int f32, hipStream_t s);
+                           int f32, hipStream_t s, const int* src = nullptr, int relu2 = 0);
 // out[t] = sum_j y[dst[t * k + j]] (+ extra[t])
 void launch_gather_sum(const void* y, const int* dst, int k, const void* extra, float* out, int T, int d, int f32,
                        hipStream_t s);

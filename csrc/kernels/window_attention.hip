@@ -1,6 +1,6 @@
-// Sliding-window softmax attention with grouped key / value heads over a paged cache, with an optional per-head
-// sigmoid output gate and an optional per-head logarithmic distance bias (the score of a key n positions back is
-// lowered by b1_h ln(1 + b2_h n)).
+// Sliding-window softmax attention with grouped key / value heads over a paged cache, with an optional sigmoid output
+// gate (per head or per column), an optional per-head logarithmic distance bias (the score of a key n positions back is
+// lowered by b1_h ln(1 + b2_h n)), an optional soft cap on the scores and an optional factor per cached key.
 //
 // Row r (position p of sequence row_seq[r]) sees positions max(0, p - window + 1) .. p and, with keep_first, the
 // sequence's first keep_first positions (at their true places in the cache); with a sink the softmax's denominator of
@@ -42,6 +42,13 @@ SYM_DEV void load_pair(const float* p, float& a, float& b) {
 // cache row of position kp of a sequence (block table bt): a shift and a mask for power-of-two blocks
 SYM_DEV long long cache_row(const int* __restrict__ bt, int kp, int BS, int shift) {
   return shift >= 0 ? ((long long)bt[kp >> shift] << shift) + (kp & (BS - 1)) : (long long)bt[kp / BS] * BS + kp % BS;
+}
+
+// cap tanh(s / cap); the 32-bit model takes tanhf, bf16 activations 1 - 2 / (1 + e^(2 x)) on the hardware exponential
+template <typename T>
+SYM_DEV float soft_cap(float s, float cap) {
+  if constexpr (sizeof(T) == 4) return cap * tanhf(s / cap);
+  else return cap - 2.f * cap / (1.f + __expf(2.f * s / cap));
 }
 
 // REP dot products of one key row with the REP query vectors of its head group (qs [REP][dk], fp32)
@@ -122,6 +129,15 @@ __global__ __launch_bounds__(64 * NW) void window_attn_wave_kernel(WindowAttnArg
     if (on) {
       slot = cache_row(bt, j, a.BS, a.bs_shift);
       dot_rows<T, REP>(kc + (slot * a.G + g) * a.dk, qs, a.dk, sc);
+      if (a.key_scale) {
+        const float ks = a.key_scale[slot];
+#pragma unroll
+        for (int r = 0; r < REP; ++r) sc[r] *= ks;
+      }
+      if (a.softcap > 0.f) {
+#pragma unroll
+        for (int r = 0; r < REP; ++r) sc[r] = soft_cap<T>(sc[r], a.softcap);
+      }
       if (a.bias) {
         // (the 32-bit model takes log1pf; bf16 activations the hardware logarithm, whose error is far below their rounding)
         const float dist = (float)(p - j);
@@ -223,10 +239,8 @@ __global__ __launch_bounds__(64 * NW) void window_attn_wave_kernel(WindowAttnArg
   for (int r = 0; r < REP; ++r) {
     const int h = h0 + r;
     float gate = 1.f;
-    if (a.gate) {
-      const float gv = (float)reinterpret_cast<const T*>(a.gate)[(long long)row * a.ldg + h];
-      gate = 1.f / (1.f + expf(-gv));
-    }
+    const T* gp = a.gate ? reinterpret_cast<const T*>(a.gate) + (long long)row * a.ldg + (a.gate_cols ? h * a.dv : h) : nullptr;
+    if (a.gate && !a.gate_cols) gate = 1.f / (1.f + expf(-(float)gp[0]));
     if (a.sink) {     // one more term in the denominator: exp(sink - M) with M = max(m, sink)
       const float sk = a.sink[h], M = fmaxf(m[r], sk);
       const float f = expf(m[r] - M);
@@ -238,7 +252,7 @@ __global__ __launch_bounds__(64 * NW) void window_attn_wave_kernel(WindowAttnArg
 #pragma unroll
     for (int i = 0; i < MAX_VCOLS; ++i) {
       const int c = vcol<PAIR>(lane, i);
-      if (i < nvc && c < a.dv) o[c] = (T)(acc[r][i] * inv);
+      if (i < nvc && c < a.dv) o[c] = (T)(acc[r][i] * inv * (a.gate_cols ? 1.f / (1.f + expf(-(float)gp[c])) : 1.f));
     }
   }
 }
@@ -483,7 +497,8 @@ int launch_window_attn(const WindowAttnArgs& args, int f32, int impl, hipStream_
   a.bs_shift = -1;
   for (int b = 0; b < 31; ++b)
     if (a.BS == 1 << b) a.bs_shift = b;
-  if (impl >= 1 && !f32 && a.tiles && a.cu_q && a.ntiles > 0 && a.dk == a.dv && a.ntiles <= 65535 * 16) {
+  const bool plain = !a.gate_cols && !a.key_scale && a.softcap <= 0.f;   // (what the tiled kernel has no code for)
+  if (impl >= 1 && plain && !f32 && a.tiles && a.cu_q && a.ntiles > 0 && a.dk == a.dv && a.ntiles <= 65535 * 16) {
     const int rw = impl == 2 ? 8 : 4;
     switch (a.dk) {
       case 32: launch_tile<32>(a, rw, s); return 1;
