@@ -1,5 +1,5 @@
 #!/usr/bin/env python3
-"""Prefill and decode throughput of a Bozevik, Lemunex, Komazen, Dalalix or Beletar stack beside the closest Llama /
+"""Prefill and decode throughput of a Bozevik, Lemunex, Komazen, Dalalix, Beletar or Bekedra stack beside the closest Llama /
 Mixtral stack of equal size.
 
 Random weights, layer shapes of real models, a few layers each (throughput per layer is what is compared; the
@@ -133,6 +133,27 @@ def _beletar_pairs():
     }
 
 
+def _bekedra_pairs():
+    """Bekedra stacks (rotary attention with soft cap, sink and gate between attention whose values are its keys; squared-ReLU
+    experts of two matrices, one and a half times as wide as the gated ones so that the expert parameters are equal) beside the
+    Mixtral stack of the same width, head count and expert count, and beside the Dalalix stack (the closest model with routed
+    experts over an fp32 stream)."""
+    from symmetry_amd.models.config import ModelConfig, bekedra_stack, dalalix_stack
+
+    kw = dict(max_position=8192, bos_token_id=32000, eos_token_ids=(32001, 32002))
+    small = bekedra_stack("bekedra-w2048", 32768, 2048, "RKRK", heads=16, kv_heads=4, dim=128, experts=16, top=4,
+                          expert_ff=2304, embed_scale=8.0, **kw)
+    return {
+        "w2048": (small, ModelConfig("mixtral-w2048", 32768, 2048, 1536, 4, 16, 4, num_experts=16, top_k=4, **kw)),
+        "w4096": (bekedra_stack("bekedra-w4096", 32768, 4096, "RKRK", heads=32, kv_heads=8, dim=128, experts=8, top=2,
+                                expert_ff=21504, embed_scale=8.0, **kw),
+                  ModelConfig("mixtral-w4096", 32768, 4096, 14336, 4, 32, 8, num_experts=8, top_k=2, **kw)),
+        "moe-w2048": (small, dalalix_stack("dalalix-w2048", 32768, 2048, "BPCC", heads=16, kv_heads=4, dim=128, experts=16,
+                                           top=4, expert_ff=1536, window=1024, keep_first=4, groups=4, keep=2, streams=4,
+                                           buckets=65521, conv=4, mem_heads=8, mem_dim=128, mem_vdim=256, **kw)),
+    }
+
+
 def measure(mcfg, prompts: int, plen: int, steps: int, reps: int = 3) -> dict:
     import torch
 
@@ -184,12 +205,12 @@ def main(argv=None) -> int:
     ap.add_argument("--prompts", type=int, default=8)
     ap.add_argument("--prompt-len", type=int, default=1024)
     ap.add_argument("--decode-steps", type=int, default=64)
-    ap.add_argument("--only", default="", help="bozevik | lemunex | komazen | dalalix | beletar | baseline: one side only (profiling)")
-    ap.add_argument("--design", default="bozevik", choices=("bozevik", "lemunex", "komazen", "dalalix", "beletar"),
+    ap.add_argument("--only", default="", help="bozevik | lemunex | komazen | dalalix | beletar | bekedra | baseline: one side only (profiling)")
+    ap.add_argument("--design", default="bozevik", choices=("bozevik", "lemunex", "komazen", "dalalix", "beletar", "bekedra"),
                     help="the family measured")
     a = ap.parse_args(argv)
     pairs = {"bozevik": _pairs, "lemunex": _lemunex_pairs, "komazen": _komazen_pairs, "dalalix": _dalalix_pairs,
-             "beletar": _beletar_pairs}[a.design]()
+             "beletar": _beletar_pairs, "bekedra": _bekedra_pairs}[a.design]()
     ratios = {}
     for size in a.sizes.split(","):
         if size not in pairs:     # (not every design has every size)

@@ -215,8 +215,11 @@ struct WindowAttnArgs {
   const int* cu_q;
   int ntiles;
 };
-// Returns the implementation used: 0 = one wave per (row, head) (all shapes, both dtypes), 1 = tiled MFMA (bf16).
+// Returns the implementation used: 0 = one wave per (row, head) (all shapes, both dtypes), 1 = tiled MFMA (bf16), 2 = the
+// causal prompt kernel of prompt_attention.hip (bf16).  impl 0: the first only; 3: not the last
 int launch_window_attn(const WindowAttnArgs& a, int f32, int impl, hipStream_t s);
+// prompt_attention.hip: causal rows in the packed prompt form, bf16, dk = dv in 32, 48, .. 128; false: not for these arguments
+bool launch_prompt_attn(const WindowAttnArgs& a, hipStream_t s);
 
 // ---- decay_scan.hip ------------------------------------------------------------------------------------
 struct DecayScanArgs {

@@ -12,6 +12,7 @@
 // rows of the segment as the other MFMA operand), and a 128 x 128 or 256 x 256 tile kernel staged through LDS by direct loads
 // for prompt steps.  Other shapes and fp32: the all-shapes segment product of glu_moe.hip.
 #include "common.h"
+#include "direct_lds.h"
 #include "hybrid_launchers.h"
 #include "latent_launchers.h"
 #include "wave_dot.h"
@@ -219,18 +220,39 @@ __global__ __launch_bounds__(64 * NW) void expert_stream_kernel(ExpertArgs a) {
       x[m] = reinterpret_cast<const bf16*>(a.x) + (long long)(a.src ? a.src[r] : r) * K + 8 * hq;
       acc[m] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-#pragma unroll 8
-    for (int c = 32 * wave; c < K; c += 32 * NW) {
-      const u32x4 wv = ld_nt16(w + c);
-      Pack8 wf;
-      wf.w = wv;
+    // 64 elements of every weight row per step: whole 128-byte lines
+    constexpr int U = MT == 1 ? 4 : 2;
+    int c = 64 * wave;
+    for (; c + 64 * NW * (U - 1) + 64 <= K; c += 64 * NW * U) {
+      Pack8 wf[U][2];
 #pragma unroll
-      for (int m = 0; m < MT; ++m) {
-        Pack8 xf;
-        xf.u = *reinterpret_cast<const uint4*>(x[m] + c);
-        acc[m] = mfma16(wf.v, xf.v, acc[m]);     // lane: row j, outputs n0 + 4 hq + 0..3
-      }
+      for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int v = 0; v < 2; ++v) wf[u][v].w = ld_nt16(w + c + 64 * NW * u + 32 * v);
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int v = 0; v < 2; ++v)
+#pragma unroll
+          for (int m = 0; m < MT; ++m) {
+            Pack8 xf;
+            xf.u = *reinterpret_cast<const uint4*>(x[m] + c + 64 * NW * u + 32 * v);
+            acc[m] = mfma16(wf[u][v].v, xf.v, acc[m]);     // lane: row j, outputs n0 + 4 hq + 0..3
+          }
     }
+    for (; c < K; c += 64 * NW)
+#pragma unroll
+      for (int v = 0; v < 2; ++v) {
+        if (c + 32 * v >= K) break;
+        Pack8 wf;
+        wf.w = ld_nt16(w + c + 32 * v);
+#pragma unroll
+        for (int m = 0; m < MT; ++m) {
+          Pack8 xf;
+          xf.u = *reinterpret_cast<const uint4*>(x[m] + c + 32 * v);
+          acc[m] = mfma16(wf.v, xf.v, acc[m]);
+        }
+      }
 #pragma unroll
     for (int m = 0; m < MT; ++m) *reinterpret_cast<f32x4*>(&part[wave][m * 256 + j * 16 + 4 * hq]) = acc[m];
     __syncthreads();
@@ -249,10 +271,6 @@ __global__ __launch_bounds__(64 * NW) void expert_stream_kernel(ExpertArgs a) {
 // global -> LDS loads.  LDS rows are 128 B with the 16-byte chunk c stored at c ^ ((row >> 1) & 7) (swizzled on the load's
 // source), so fragment reads do not conflict.  The tile list is walked on the device: a slot past the last tile exits before
 // any barrier.  K % 64 == 0.
-SYM_DEV void direct_load16(const bf16* src, char* lds) {
-  __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src,
-                                   (__attribute__((address_space(3))) void*)lds, 16, 0, 0);
-}
 SYM_DEV int chunk_swz(int row) { return (row >> 1) & 7; }
 
 template <int BM, int BN, int WR, int WC>
@@ -292,12 +310,13 @@ __global__ __launch_bounds__(64 * WR * WC) void expert_tile_kernel(ExpertArgs a)
     const int row = 8 * (NWV * i + wave) + (lane >> 3), ch = (lane & 7) ^ chunk_swz(row);
     bsrc[i] = reinterpret_cast<const bf16*>(a.W) + ((long long)e * N + min(n0 + row, N - 1)) * K + 8 * ch;
   }
+  const unsigned int lds0 = lds_address(smem) + __builtin_amdgcn_readfirstlane(wave) * 1024;
   auto stage = [&](int kt, int buf) {
-    char* base = smem + buf * STAGE;
+    const unsigned int base = lds0 + buf * STAGE;
 #pragma unroll
-    for (int i = 0; i < AL; ++i) direct_load16(asrc[i] + kt * 64, base + (NWV * i + wave) * 1024);
+    for (int i = 0; i < AL; ++i) direct_load16(asrc[i] + kt * 64, base + NWV * i * 1024);
 #pragma unroll
-    for (int i = 0; i < BL; ++i) direct_load16(bsrc[i] + kt * 64, base + AB + (NWV * i + wave) * 1024);
+    for (int i = 0; i < BL; ++i) direct_load16(bsrc[i] + kt * 64, base + AB + NWV * i * 1024);
   };
   f32x4 acc[NS][MS];
 #pragma unroll
@@ -308,7 +327,7 @@ __global__ __launch_bounds__(64 * WR * WC) void expert_tile_kernel(ExpertArgs a)
   const int nk = K / 64;
   stage(0, 0);
   for (int kt = 0; kt < nk; ++kt) {
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    wait_direct_loads();
     __syncthreads();      // stage kt has landed for every wave, and every wave is done reading the other stage
     if (kt + 1 < nk) stage(kt + 1, (kt + 1) & 1);
     const char* A = smem + (kt & 1) * STAGE;
@@ -413,10 +432,10 @@ int launch_expert_linear(const ExpertArgs& a, int f32, int impl, hipStream_t s) 
   const bool mfma = !f32 && aligned16(a.x) && aligned16(a.W) && aligned16(a.y);
   const int per = (a.R + a.E - 1) / a.E;      // rows per expert if they are spread evenly
   const bool stream = mfma && a.K % 32 == 0 && a.E <= 65535, tile = mfma && a.K % 64 == 0;
-  if (impl < 0) impl = stream && per <= 64 ? 1 : (tile ? (per >= 512 && a.N >= 256 ? 3 : 2) : (stream ? 1 : 0));
+  if (impl < 0) impl = stream && (per <= 8 || !tile) ? 1 : (tile ? (per >= 512 && a.N >= 256 ? 3 : 2) : (stream ? 1 : 0));
   if (impl == 1 && stream) {
     dim3 grid((a.N + 15) / 16, a.E);
-    if (per <= 8) expert_stream_kernel<1, 4><<<grid, 256, 0, s>>>(a);
+    if (per <= 8) expert_stream_kernel<1, 8><<<grid, 512, 0, s>>>(a);      // (8 waves: 31 us, 4 waves: 33 us at 16 x 2304 x 2048)
     else if (per <= 24) expert_stream_kernel<2, 4><<<grid, 256, 0, s>>>(a);
     else expert_stream_kernel<4, 4><<<grid, 256, 0, s>>>(a);
     return 1;
