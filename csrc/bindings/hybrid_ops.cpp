@@ -184,7 +184,8 @@ void qkv_rope_cache(const Tensor& z, const OptTensor& bias, int64_t H, int64_t G
 int64_t window_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache, const Tensor& block_tables,
                     const Tensor& row_seq, const Tensor& positions, int64_t window, double scale, const OptTensor& gate,
                     Tensor& out, const OptTensor& tiles, const OptTensor& cu_q, int64_t impl, const OptTensor& bias,
-                    int64_t keep_first, const OptTensor& sink, double softcap, const OptTensor& key_scale) {
+                    int64_t keep_first, const OptTensor& sink, double softcap, const OptTensor& key_scale,
+                    const OptTensor& part_o, const OptTensor& part_ml, const OptTensor& counters, int64_t part_keys) {
   const int f32 = act(q, "q");
   same_act(k_cache, f32, "k_cache");
   same_act(v_cache, f32, "v_cache");
@@ -225,6 +226,18 @@ int64_t window_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cach
     a.key_scale = ptr<float>(*key_scale);
   }
   a.softcap = (float)softcap;
+  if (part_o.has_value()) {
+    TORCH_CHECK(part_ml.has_value() && counters.has_value() && part_keys >= 32, "window_attn: part_o without part_ml / counters");
+    dtype(*part_o, at::kFloat, "part_o");
+    dtype(*part_ml, at::kFloat, "part_ml");
+    dtype(*counters, at::kInt, "counters");
+    const int64_t span = (int64_t)a.max_blocks * a.BS, parts = (span + part_keys - 1) / part_keys;
+    TORCH_CHECK(part_keys < (1LL << 30) && part_o->numel() >= (int64_t)a.T * a.H * parts * a.dv &&
+                    part_ml->numel() >= (int64_t)a.T * a.H * parts * 2 && counters->numel() >= (int64_t)a.T * a.G,
+                "window_attn: part_o [T, H, parts, dv], part_ml [T, H, parts, 2], counters [T, G]");
+    a.part_o = ptr<float>(*part_o), a.part_ml = ptr<float>(*part_ml), a.counters = ptr<int>(*counters);
+    a.part_keys = (int)part_keys, a.max_parts = (int)parts;
+  }
   TORCH_CHECK(keep_first >= 0 && keep_first < (1LL << 30), "window_attn: keep_first");
   a.keep_first = (int)keep_first;
   if (tiles.has_value() && cu_q.has_value()) {
@@ -1094,7 +1107,8 @@ TORCH_LIBRARY(symmetry_amd_hybrid, m) {
   m.def(
       "window_attn(Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor row_seq, Tensor positions, "
       "int window, float scale, Tensor? gate, Tensor(a!) out, Tensor? tiles, Tensor? cu_q, int impl, Tensor? bias, "
-      "int keep_first, Tensor? sink, float softcap=0., Tensor? key_scale=None) -> int",
+      "int keep_first, Tensor? sink, float softcap=0., Tensor? key_scale=None, Tensor(b!)? part_o=None, "
+      "Tensor(c!)? part_ml=None, Tensor(d!)? counters=None, int part_keys=0) -> int",
       &window_attn);
   m.def(
       "decay_scan(int mode, Tensor q, Tensor k, Tensor v, Tensor dz, Tensor dbias, Tensor? rate, float tau, Tensor? skip, "

@@ -214,12 +214,21 @@ struct WindowAttnArgs {
   const int* tiles;
   const int* cu_q;
   int ntiles;
+  // single rows in ranges of part_keys keys (split_attention.hip), or null: partial sums [T][G][max_parts][H / G][dv] and
+  // (maximum, sum) [T][G][max_parts][H / G][2]; arrival counters [T][G], zero between launches
+  float* part_o;
+  float* part_ml;
+  int* counters;
+  int part_keys, max_parts;
 };
 // Returns the implementation used: 0 = one wave per (row, head) (all shapes, both dtypes), 1 = tiled MFMA (bf16), 2 = the
-// causal prompt kernel of prompt_attention.hip (bf16).  impl 0: the first only; 3: not the last
+// causal prompt kernel of prompt_attention.hip (bf16), 3 = the key ranges of split_attention.hip (bf16).  impl 0: the first
+// only; 3: the first two
 int launch_window_attn(const WindowAttnArgs& a, int f32, int impl, hipStream_t s);
 // prompt_attention.hip: causal rows in the packed prompt form, bf16, dk = dv in 32, 48, .. 128; false: not for these arguments
 bool launch_prompt_attn(const WindowAttnArgs& a, hipStream_t s);
+// split_attention.hip: single rows with part_o set, causal, bf16, dk = dv in 32, 48, .. 128, H / G <= 16; false: not for these
+bool launch_split_attn(const WindowAttnArgs& a, hipStream_t s);
 
 // ---- decay_scan.hip ------------------------------------------------------------------------------------
 struct DecayScanArgs {

@@ -11,43 +11,19 @@
 //
 // Softmax statistics are fp32.  Without a cap: running maximum (one cross-lane step per tile), sums combined at the end.  With
 // a cap c <= 60 the scores lie in [-c, c], so e^s needs no maximum: p = 2^(c' - 2 c' / (1 + 2^(2 s log2(e) / c))), c' = c log2 e.
-#include "common.h"
-#include "direct_lds.h"
+#include "attn_tiles.h"
 #include "hybrid_launchers.h"
 
 namespace {
 
-constexpr float LOG2E = 1.44269504088896341f;
 constexpr float MAX_CAP = 60.f;      // e^60 times any number of keys and e^-60 are well inside fp32 and bf16
 constexpr int PW = 4, ROWS = 32 * PW;
 
-typedef short s16x4 __attribute__((ext_vector_type(4)));
-
 SYM_DEV f32x16 mfma32(bf16x8 a, bf16x8 b, f32x16 c) { return __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0); }
-
-// transpose read: the 16 lanes of a group hand in 8-byte pieces of a 4 x 16 matrix (lane l: row l / 4, columns 4 (l % 4) ..);
-// lane i receives column i
-SYM_DEV uint2 read_tr(const char* lds) {
-  const s16x4 v = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)lds);
-  return __builtin_bit_cast(uint2, v);
-}
-
-// 16-byte chunks per LDS row of a head of D entries (a power of two), and the row's XOR
-constexpr int chunks(int D) { return D <= 32 ? 4 : (D <= 64 ? 8 : 16); }
-template <int CH>
-SYM_DEV int swz(int r) {
-  if constexpr (CH == 16) return 4 * (r & 3) + ((r >> 2) & 3);
-  else if constexpr (CH == 8) return 4 * ((r >> 1) & 1) + ((r >> 2) & 3);
-  else return (r >> 2) & 3;
-}
-
-SYM_DEV long long cache_row(const int* __restrict__ bt, int kp, int BS, int shift) {
-  return shift >= 0 ? ((long long)bt[kp >> shift] << shift) + (kp & (BS - 1)) : (long long)bt[kp / BS] * BS + kp % BS;
-}
 
 template <int D, bool CAP, bool KEYV, bool ONE>
 __global__ __launch_bounds__(64 * PW, 2) void prompt_attn_kernel(WindowAttnArgs a) {
-  constexpr int CH = chunks(D), KD = D / 16, VT = (D + 31) / 32, TILE = 64 * CH * 16;   // bytes of a staged tile
+  constexpr int CH = row_chunks(D), KD = D / 16, VT = (D + 31) / 32, TILE = 64 * CH * 16;   // bytes of a staged tile
   constexpr int NL = CH / PW;                          // direct loads per wave and tile (64 / CH rows each)
   constexpr int STAGE = (KEYV ? 1 : 2) * TILE + 256;   // keys, values, 64 key factors
   extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -120,8 +96,8 @@ __global__ __launch_bounds__(64 * PW, 2) void prompt_attn_kernel(WindowAttnArgs 
 #pragma unroll
     for (int e = 0; e < 16; ++e) o[i][e] = 0.f;
   float m = CAP ? 0.f : -INFINITY, l = 0.f;            // l: this lane's keys only, the two lanes of a row meet at the end
-  const float sl2 = a.scale * LOG2E;
-  const float c1 = CAP ? 2.f * sl2 / a.softcap : 0.f, c2 = CAP ? a.softcap * LOG2E : 0.f;
+  const float sl2 = a.scale * ATT_LOG2E;
+  const float c1 = CAP ? 2.f * sl2 / a.softcap : 0.f, c2 = CAP ? a.softcap * ATT_LOG2E : 0.f;
   const bool scaled = a.key_scale != nullptr;
 
   if (ONE) blk = bt[0];
@@ -239,7 +215,7 @@ __global__ __launch_bounds__(64 * PW, 2) void prompt_attn_kernel(WindowAttnArgs 
                           : nullptr;
   if (a.gate && !a.gate_cols) fac = 1.f / (1.f + expf(-(float)gp[0]));
   if (a.sink) {     // one more term in the denominator (m is in units of log2 e)
-    const float sk = a.sink[h] * LOG2E, M = fmaxf(m, sk), f = exp2f(m - M);
+    const float sk = a.sink[h] * ATT_LOG2E, M = fmaxf(m, sk), f = exp2f(m - M);
     l = l * f + exp2f(sk - M);
     fac *= f;
   }
@@ -270,7 +246,7 @@ __global__ __launch_bounds__(64 * PW, 2) void prompt_attn_kernel(WindowAttnArgs 
 
 template <int D, bool CAP, bool KEYV, bool ONE>
 void launch(const WindowAttnArgs& a, hipStream_t s) {
-  constexpr int lds = 2 * ((KEYV ? 1 : 2) * 64 * chunks(D) * 16 + 256);
+  constexpr int lds = 2 * ((KEYV ? 1 : 2) * 64 * row_chunks(D) * 16 + 256);
   static bool once = false;
   if (lds > 64 * 1024 && !once) {
     hipFuncSetAttribute(reinterpret_cast<const void*>(&prompt_attn_kernel<D, CAP, KEYV, ONE>),

@@ -497,7 +497,10 @@ int launch_window_attn(const WindowAttnArgs& args, int f32, int impl, hipStream_
   a.bs_shift = -1;
   for (int b = 0; b < 31; ++b)
     if (a.BS == 1 << b) a.bs_shift = b;
-  if (impl >= 1 && impl != 3 && !f32 && launch_prompt_attn(a, s)) return 2;
+  if (impl >= 1 && impl != 3 && !f32) {
+    if (launch_prompt_attn(a, s)) return 2;
+    if (!a.tiles && launch_split_attn(a, s)) return 3;
+  }
   const bool plain = !a.gate_cols && !a.key_scale && a.softcap <= 0.f;   // (what the tiled kernel has no code for)
   if (impl >= 1 && plain && !f32 && a.tiles && a.cu_q && a.ntiles > 0 && a.dk == a.dv && a.ntiles <= 65535 * 16) {
     const int rw = impl == 2 ? 8 : 4;

@@ -51,7 +51,7 @@ LATENT_BINDINGS = ("latent_ops.cpp",)
 # kernels, so that translation unit is linked into both libraries
 HYBRID_SO = os.path.join(PKG, "_C_hybrid.so")
 HYBRID_KERNELS = ("hybrid_rows.hip", "stream_rows.hip", "norm_rows.hip", "routed_ff.hip", "window_attention.hip", "prompt_attention.hip",
-                  "decay_scan.hip", "delta_rule.hip")
+                  "split_attention.hip", "decay_scan.hip", "delta_rule.hip")
 HYBRID_SHARED = ("glu_moe.hip",)
 HYBRID_BINDINGS = ("hybrid_ops.cpp",)
 NET_SO = os.path.join(PKG, "net", "_native.so")
@@ -113,7 +113,8 @@ def build_kernels(verbose: bool = False, force: bool = False) -> str:
     kdir = os.path.join(CSRC, "kernels")
     # (the family libraries' launcher headers are not included by these translation units)
     headers = [h for h in glob.glob(os.path.join(kdir, "*.h")) + glob.glob(os.path.join(kdir, "*.cuh"))
-               if os.path.basename(h) not in ("latent_launchers.h", "hybrid_launchers.h", "wave_dot.h", "direct_lds.h")]
+               if os.path.basename(h) not in ("latent_launchers.h", "hybrid_launchers.h", "wave_dot.h", "direct_lds.h",
+                                           "attn_tiles.h")]
     sources = sorted(s for s in glob.glob(os.path.join(kdir, "*.hip"))
                      if os.path.basename(s) not in LATENT_KERNELS + HYBRID_KERNELS)
     tinc, tlib, abi = _torch_paths()
@@ -185,11 +186,11 @@ def build_latent(verbose: bool = False, force: bool = False) -> str:
 
 
 def build_hybrid(verbose: bool = False, force: bool = False) -> str:
-    """csrc/kernels/{hybrid_rows,stream_rows,norm_rows,routed_ff,window_attention,prompt_attention,decay_scan,delta_rule,glu_moe}.hip + csrc/bindings/hybrid_ops.cpp ->
+    """csrc/kernels/{hybrid_rows,stream_rows,norm_rows,routed_ff,window_attention,prompt_attention,split_attention,decay_scan,delta_rule,glu_moe}.hip + csrc/bindings/hybrid_ops.cpp ->
     symmetry_amd/_C_hybrid.so (``torch.ops.symmetry_amd_hybrid``)."""
     os.makedirs(OBJ, exist_ok=True)
     kdir = os.path.join(CSRC, "kernels")
-    headers = [os.path.join(kdir, h) for h in ("common.h", "wave_dot.h", "direct_lds.h", "hybrid_launchers.h", "latent_launchers.h")]
+    headers = [os.path.join(kdir, h) for h in ("common.h", "wave_dot.h", "direct_lds.h", "attn_tiles.h", "hybrid_launchers.h", "latent_launchers.h")]
     tinc, tlib, abi = _torch_paths()
     jobs, objs = [], []
     for name in HYBRID_KERNELS + HYBRID_SHARED:

@@ -173,9 +173,15 @@ class BekedraLM:
             ops.qk_norm_cache(qkv, m.heads, m.kv_heads, m.dim, m.vdim, P["gq"], P["gk"], None, eps, b.slot_mapping, q,
                               cache.k[n], cache.v[n], rope=P["rope"], positions=b.positions)
         att = self._buf("att.o", (T, m.heads, m.vdim))
+        split = None
+        if not prefill and self.device.type != "cpu" and self.dtype == torch.bfloat16:
+            keys, parts = ops.window_attn_split(T, m.kv_heads, b.block_tables.shape[1] * cache.block_size)
+            split = (self._buf("att.part_o", (T, m.heads, parts, m.vdim), torch.float32),
+                     self._buf("att.part_ml", (T, m.heads, parts, 2), torch.float32),
+                     self.ws.get("att.counters", (T * m.kv_heads,), torch.int32, self.device, zeros=True), keys)
         ops.window_attn(q, cache.k[n], cache.k[n] if m.key_values else cache.v[n], b.block_tables, b.row_seq, b.positions,
                         CAUSAL, m.scale, self._cols(z, P, "g") if m.gate else None, att, b.tiles if prefill else None,
-                        b.cu_q if prefill else None, sink=P["sink"], softcap=m.softcap, key_scale=cache.ks.get(n))
+                        b.cu_q if prefill else None, sink=P["sink"], softcap=m.softcap, key_scale=cache.ks.get(n), split=split)
         return self._linear("att.out", att.view(T, m.heads * m.vdim), P["o"])
 
     def _routed(self, P: dict, h: torch.Tensor):

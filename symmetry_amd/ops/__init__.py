@@ -781,7 +781,7 @@ WINDOW_ATTN_IMPL = 0 if os.environ.get("SYMMETRY_WINDOW_ATTN", "auto") == "wave"
 
 
 def window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, window, scale, gate, out, tiles=None, cu_q=None,
-                impl=None, bias=None, keep_first=0, sink=None, softcap=0.0, key_scale=None):
+                impl=None, bias=None, keep_first=0, sink=None, softcap=0.0, key_scale=None, split=None):
     """Softmax attention of q [T, H, dk] over the paged caches: row r sees positions max(0, p - window + 1) .. p of
     sequence row_seq[r] (p = positions[r]) and, with ``keep_first``, the sequence's first keep_first positions; query
     head h reads key / value head h // (H / G); scores and weights fp32.  ``gate`` [T, H] or [T, H dv] (a view): head outputs, or
@@ -790,14 +790,26 @@ def window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, window, s
     the score of a key at distance n = p - j is lowered by bias[0, h] * ln(1 + bias[1, h] * n).  ``sink`` [H] fp32: the
     softmax's denominator of head h also holds exp(sink[h]) (a logit without a key or a value, not scaled or capped).
     ``key_scale`` [NB, BS] fp32: the scores of a key are multiplied by its cache row's number; ``softcap`` c > 0: scores
-    become c tanh(s / c) (before the distance bias).  ``v_cache`` may be ``k_cache`` itself."""
+    become c tanh(s / c) (before the distance bias).  ``v_cache`` may be ``k_cache`` itself.  ``split``
+    (single rows: decode steps): (part_o, part_ml, counters, part_keys), workspace for walking a row's keys in ranges of
+    part_keys (``window_attn_split``) side by side; the counters are zero before and after every launch."""
     if _gpu(q):
         return _hyb().window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, int(window), float(scale), gate,
                                   out, tiles, cu_q, WINDOW_ATTN_IMPL if impl is None else int(impl), bias,
-                                  int(keep_first), sink, float(softcap), key_scale)
+                                  int(keep_first), sink, float(softcap), key_scale, *(split or ()))
     reference.window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, window, scale, gate, out, bias,
                           keep_first, sink, softcap, key_scale)
     return 0
+
+
+def window_attn_split(rows: int, groups: int, span: int, target_wgs: int = 512, max_parts: int = 64):
+    """(part_keys, parts) for walking ``span`` keys of ``rows`` single rows with ``groups`` key / value heads in ranges side by
+    side: ranges as short as one step of a workgroup's waves (128 keys) as long as that makes no more than ``target_wgs``
+    workgroups, and no more than ``max_parts`` of them."""
+    keys = 128
+    while rows * groups * (span // keys) > target_wgs or -(-span // keys) > max_parts:
+        keys *= 2
+    return keys, -(-span // keys)
 
 
 DECAY_CHANNEL_GATE, DECAY_STEP_SIZE, DECAY_LOG_GATES = 0, 1, 2

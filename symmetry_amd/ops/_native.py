@@ -85,7 +85,7 @@ _hybrid_loaded = False
 
 
 def hybrid_ops():
-    """``torch.ops.symmetry_amd_hybrid`` (loaded once; built first if the library is missing: ten translation units,
+    """``torch.ops.symmetry_amd_hybrid`` (loaded once; built first if the library is missing: eleven translation units,
     about a minute).  Raises if it cannot be built or loaded: no eager fallback on the device."""
     global _hybrid_loaded
     with _lock:
