@@ -21,11 +21,13 @@ v / sqrt(mean(v^2) + eps) * g)::
 Caches belong to a layer RUN: a looped layer has planes per pass.  Nothing else is kept per sequence, so the model needs no
 state slots and cached prompt prefixes are adopted as they are.  Every bf16 projection that reads h is one row block of one
 fused weight (a single library GEMM); the kernels take column ranges as views.  Step launches per layer run:
-    attention:    GEMM q | k, qk_row_norm_cache, window_attn (key scales), GEMM W_o
+    attention:    GEMM q | k, qk_row_norm_cache, window_attn (key scales; decode: key ranges), GEMM W_o
     attention_2:  GEMM q | k | v | gate, qk_norm_cache (rotary), window_attn (soft cap, sink, gate), GEMM W_o
     ff:           route_topk, expert_linear (gathers its rows, squared ReLU), expert_linear
     residual_routed_norm (stream + mixer + weighted expert rows + the next pass's vector, and the next layer's h)
-All intermediates live in the preallocated Workspace, so decode steps are hipGraph-capturable.
+All intermediates live in the preallocated Workspace, so decode steps are hipGraph-capturable.  In decode steps the experts
+(bound by their weights' traffic) run on a second stream beside the attention (bound by latency): two branches of the graph,
+joined in front of the sum.
 
 fp32 in both serving dtypes: the stream, norm statistics, rotary angles, temperatures, attention scores / weights / sink /
 cap, router logits and weights.  ``dtype=torch.float32`` runs every product in true 32-bit as well.
@@ -85,6 +87,7 @@ class BekedraLM:
         self.last_ids = torch.zeros(MAX_STEP_SEQS, dtype=torch.int32, device=self.device)
         self.last_logits = None
         self.layer_outputs: list | None = None   # set to a list: every forward appends the stream after each layer run
+        self.side = torch.cuda.Stream(self.device) if self.device.type != "cpu" else None
         cfg = self.cfg
         max_pos = min(cfg.max_position, max_decode_ctx or cfg.max_position)
         self._rope: dict = {}
@@ -213,12 +216,21 @@ class BekedraLM:
         ops.embed_scale(b.input_ids, self.embed, cfg.embed_scale, x, src, self.last_ids if src is not None else None)
         P0, step = self.runs[0]
         ops.residual_routed_norm(x, None, None, None, None, 0, step, P0["norm1"], eps, h)
+        side, main = (None, None) if prefill or self.side is None else (self.side, torch.cuda.current_stream(self.device))
         for n, (P, _) in enumerate(self.runs):
-            att = self._attention(n, P, b, cache, h)
             y = dst = wts = None
+            top = 0
             if P["mlp"] is not None:
-                y, dst, wts = self._routed(P, h)
-            top = P["mlp"].top if P["mlp"] is not None else 0
+                top = P["mlp"].top
+                if side is None:
+                    y, dst, wts = self._routed(P, h)
+                else:      # both sublayers read h: two branches of the step's graph
+                    side.wait_stream(main)
+                    with torch.cuda.stream(side):
+                        y, dst, wts = self._routed(P, h)
+            att = self._attention(n, P, b, cache, h)
+            if top and side is not None:
+                main.wait_stream(side)
             nxt, step = self.runs[n + 1] if n + 1 < len(self.runs) else (None, None)
             w, out = (nxt["norm1"], h) if nxt is not None else (None, None)
             if self.layer_outputs is not None:

@@ -745,3 +745,49 @@ def test_prompt_kernel_on_unequal_runs(D, BS):
                 s = O.soft_cap(s, cap)
             want = O.mix_values(O.causal_softmax(s, sink.double()), V, H)[c:]
             close(out[int(cu[i]):int(cu[i]) + n].reshape(n, -1), want, 1.5e-2)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("D", [32, 48, 64, 80, 96, 112, 128])
+@pytest.mark.parametrize("keys", [None, 32, 64, 256, 4096])
+def test_key_ranges_of_single_rows(D, keys):
+    """Decode attention by key ranges: contexts of one key up to many ranges, last ranges of one key, in blocks of 16, 24 and
+    64, one to eight query heads per key head; against the oracle, twice through the same workspace (the arrival counters are
+    back at zero)."""
+    say("op split attention", D, keys)
+    torch.manual_seed(D)
+    for H, G, BS, cap, same, per_col in ((8, 4, 64, 6.0, False, True), (4, 4, 16, 0.0, True, False), (8, 1, 24, 80.0, False, False)):
+        ctx = [1, 2, 31, 32, 33, 64, 65, 128, 129, 300, 1025]
+        T, mb = len(ctx), -(-max(ctx) // BS)
+        bt = (torch.randperm(T * mb) + 1).view(T, mb).int()
+        k, v = torch.randn(T * mb + 1, BS, G, D).to(BF16), torch.randn(T * mb + 1, BS, G, D).to(BF16)
+        ks = torch.rand(T * mb + 1, BS) + 0.3 if same else None
+        q, sink = (2.0 * torch.randn(T, H, D)).to(BF16), torch.randn(H)
+        gate = torch.randn(T, H * D if per_col else H).to(BF16)
+        pk, parts = ops.window_attn_split(T, G, mb * BS)
+        if keys:
+            pk, parts = keys, -(-mb * BS // keys)
+        ws = (torch.full((T, H, parts, D), float("nan"), device="cuda"), torch.full((T, H, parts, 2), float("nan"), device="cuda"),
+              torch.zeros(T * G, dtype=torch.int32, device="cuda"), pk)
+        kd = k.cuda()
+        args = [q.cuda(), kd, kd if same else v.cuda(), bt.cuda(), torch.arange(T).int().cuda(),
+                (torch.tensor(ctx) - 1).int().cuda()]
+        for _ in range(2):
+            out = torch.full((T, H, D), 9.0, dtype=BF16, device="cuda")
+            impl = ops.window_attn(*args, CAUSAL, D ** -0.5, gate.cuda(), out, sink=sink.cuda(), softcap=cap,
+                                   key_scale=None if ks is None else ks.cuda(), split=ws)
+            assert impl == (3 if parts <= 64 else 0)
+            assert int(ws[2].abs().max()) == 0
+            for t, n in enumerate(ctx):
+                idx = torch.arange(n)
+                at = bt[t][idx // BS].long(), idx % BS
+                K, V = k[at].double(), (k if same else v)[at].double()
+                full = torch.zeros(n, H, D, dtype=F64)
+                full[-1] = q[t].double()
+                s = O.causal_scores(full, K, D ** -0.5)
+                if ks is not None:
+                    s = s * ks[at].double()
+                if cap:
+                    s = O.soft_cap(s, cap)
+                want = O.mix_values(O.causal_softmax(s, sink.double()), V, H)[-1].view(H, D)
+                close(out[t], want * torch.sigmoid(gate[t].double()).view(H, -1), 1.5e-2)
