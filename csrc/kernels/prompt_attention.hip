@@ -221,6 +221,21 @@ __global__ __launch_bounds__(64 * PW, 2) void prompt_attn_kernel(WindowAttnArgs 
   }
   const float inv = fac / l;
   bf16* out = reinterpret_cast<bf16*>(a.out) + ((long long)my_row * a.H + h) * D;
+  bf16x4 gv[VT][4];      // all gates in flight before the first store (which the loads could not pass)
+  if (a.gate_cols) {
+    const bool vec = (a.ldg & 3) == 0 && (reinterpret_cast<uintptr_t>(a.gate) & 7) == 0;
+#pragma unroll
+    for (int dt = 0; dt < VT; ++dt)
+#pragma unroll
+      for (int e4 = 0; e4 < 4; ++e4) {
+        const int c = 32 * dt + 8 * e4 + 4 * hi;
+        if (D % 32 && c >= D) continue;
+        if (vec) gv[dt][e4] = *reinterpret_cast<const bf16x4*>(gp + c);
+        else
+#pragma unroll
+          for (int u = 0; u < 4; ++u) gv[dt][e4][u] = gp[c + u];
+      }
+  }
 #pragma unroll
   for (int dt = 0; dt < VT; ++dt)
 #pragma unroll
@@ -228,17 +243,11 @@ __global__ __launch_bounds__(64 * PW, 2) void prompt_attn_kernel(WindowAttnArgs 
       const int c = 32 * dt + 8 * e4 + 4 * hi;
       if (D % 32 && c >= D) continue;
       bf16x4 w;
-      if (a.gate_cols) {
-        bf16x4 gv;
-        if ((a.ldg & 3) == 0 && (reinterpret_cast<uintptr_t>(a.gate) & 7) == 0) gv = *reinterpret_cast<const bf16x4*>(gp + c);
-        else
 #pragma unroll
-          for (int u = 0; u < 4; ++u) gv[u] = gp[c + u];
-#pragma unroll
-        for (int u = 0; u < 4; ++u) w[u] = (bf16)(o[dt][4 * e4 + u] * inv / (1.f + __expf(-(float)gv[u])));
-      } else {
-#pragma unroll
-        for (int u = 0; u < 4; ++u) w[u] = (bf16)(o[dt][4 * e4 + u] * inv);
+      for (int u = 0; u < 4; ++u) {
+        float v = o[dt][4 * e4 + u] * inv;
+        if (a.gate_cols) v *= __builtin_amdgcn_rcpf(1.f + __expf(-(float)gv[dt][e4][u]));
+        w[u] = (bf16)v;
       }
       *reinterpret_cast<bf16x4*>(out + c) = w;
     }

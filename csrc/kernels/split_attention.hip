@@ -4,10 +4,11 @@
 //
 // Four waves, 32 keys per wave and step.  A step's key and value rows go to the wave's own LDS by direct loads (KEYV: the
 // values are the keys, one set of rows serves both products); the workgroups that share a CU cover each other's loads (a second
-// stage per wave halves their number and measured slower: 64 rows x 1060 keys 60 us against 40 us).  Scores are S^T = K Q^T on v_mfma_f32_16x16x32_bf16 (16 query heads as columns), the weights go back as they lie
-// into O^T = V^T P^T with transposed value fragments from the row-major rows (LDS transpose read).  Waves meet in LDS, ranges
-// through write-through partial results and an arrival counter per (row, group): the workgroup that arrives last sums them in
-// order, writes the output and sets the counter back to zero (nobody waits).  Softmax statistics and partial sums are fp32.
+// stage per wave halves their number and measured slower: 64 rows x 1060 keys 60 us against 40 us).  Scores are S^T = K Q^T on
+// v_mfma_f32_16x16x32_bf16 (16 query heads as columns), the weights go back as they lie into O^T = V^T P^T with transposed value
+// fragments from the row-major rows (LDS transpose read).  Waves meet in LDS, ranges through write-through partial results and
+// an arrival counter per (row, group): the workgroup that arrives last sums them in order, writes the output and sets the
+// counter back to zero (nobody waits).  Softmax statistics and partial sums are fp32.
 #include "attn_tiles.h"
 #include "hybrid_launchers.h"
 

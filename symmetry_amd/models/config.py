@@ -1516,8 +1516,8 @@ def known_models() -> list[str]:
 
 def from_config_json(cfg: dict, name: str = "hf", shapes: dict | None = None):
     """The model configuration of a checkpoint directory's config.json: the design is chosen by its
-    ``architecture`` key (Bozevik, Lemunex, Komazen, Dalalix, Beletar, Bekedra), otherwise the HuggingFace Llama / Mixtral keys.  ``shapes``:
-    the checkpoint's tensor shapes, for designs that leave some sizes to them."""
+    ``architecture`` key (Bozevik, Lemunex, Komazen, Dalalix, Beletar, Bekedra), otherwise the HuggingFace Llama / Mixtral
+    keys.  ``shapes``: the checkpoint's tensor shapes, for designs that leave some sizes to them."""
     if cfg.get("architecture") == "Bozevik":
         return bozevik_from_config(cfg, name)
     if cfg.get("architecture") == "Lemunex":

@@ -784,15 +784,16 @@ def window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, window, s
                 impl=None, bias=None, keep_first=0, sink=None, softcap=0.0, key_scale=None, split=None):
     """Softmax attention of q [T, H, dk] over the paged caches: row r sees positions max(0, p - window + 1) .. p of
     sequence row_seq[r] (p = positions[r]) and, with ``keep_first``, the sequence's first keep_first positions; query
-    head h reads key / value head h // (H / G); scores and weights fp32.  ``gate`` [T, H] or [T, H dv] (a view): head outputs, or
-    their entries one by one, are multiplied by sigmoid(gate).  ``tiles`` / ``cu_q``: the packed prompt form (64-row query tiles), for the tiled
-    kernel.  Returns the implementation used (0: one wave per (row, head), every shape; 1: tiled; 2: causal prompt kernel).  ``bias`` [2, H] fp32:
-    the score of a key at distance n = p - j is lowered by bias[0, h] * ln(1 + bias[1, h] * n).  ``sink`` [H] fp32: the
-    softmax's denominator of head h also holds exp(sink[h]) (a logit without a key or a value, not scaled or capped).
-    ``key_scale`` [NB, BS] fp32: the scores of a key are multiplied by its cache row's number; ``softcap`` c > 0: scores
-    become c tanh(s / c) (before the distance bias).  ``v_cache`` may be ``k_cache`` itself.  ``split``
-    (single rows: decode steps): (part_o, part_ml, counters, part_keys), workspace for walking a row's keys in ranges of
-    part_keys (``window_attn_split``) side by side; the counters are zero before and after every launch."""
+    head h reads key / value head h // (H / G); scores and weights fp32.  ``gate`` [T, H] or [T, H dv] (a view): head
+    outputs, or their entries one by one, are multiplied by sigmoid(gate).  ``tiles`` / ``cu_q``: the packed prompt form
+    (64-row query tiles), for the tiled kernels.  Returns the implementation used (0: one wave per (row, head), every
+    shape; 1: tiled; 2: causal prompt kernel; 3: key ranges of single rows).  ``bias`` [2, H] fp32: the score of a key at
+    distance n = p - j is lowered by bias[0, h] * ln(1 + bias[1, h] * n).  ``sink`` [H] fp32: the softmax's denominator of
+    head h also holds exp(sink[h]) (a logit without a key or a value, not scaled or capped).  ``key_scale`` [NB, BS] fp32:
+    the scores of a key are multiplied by its cache row's number; ``softcap`` c > 0: scores become c tanh(s / c) (before
+    the distance bias).  ``v_cache`` may be ``k_cache`` itself.  ``split`` (single rows: decode steps): (part_o, part_ml,
+    counters, part_keys), workspace for walking a row's keys in ranges of part_keys (``window_attn_split``) side by side;
+    the counters are zero before and after every launch."""
     if _gpu(q):
         return _hyb().window_attn(q, k_cache, v_cache, block_tables, row_seq, positions, int(window), float(scale), gate,
                                   out, tiles, cu_q, WINDOW_ATTN_IMPL if impl is None else int(impl), bias,

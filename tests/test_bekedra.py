@@ -628,7 +628,8 @@ def test_router_and_experts(device, dtype, T, shape):
     if 1 < k < E:
         W["m.router.b"][E - 1], W["m.router.b"][0] = -1e3, 1e3
     for e in range(E):
-        W[f"m.e{e}.up"], W[f"m.e{e}.down"] = (torch.randn(ff, d) * d ** -0.5).to(dtype), (torch.randn(d, ff) * ff ** -0.5).to(dtype)
+        W[f"m.e{e}.up"] = (torch.randn(ff, d) * d ** -0.5).to(dtype)
+        W[f"m.e{e}.down"] = (torch.randn(d, ff) * ff ** -0.5).to(dtype)
     Wd = {n: v.double() for n, v in W.items()}
     ids_w, wts_w = O.route(Wd, "m.", k, h.double())
     i32 = torch.int32
