@@ -200,7 +200,7 @@ SYM_DEV float relu2f(float v) {
 }
 
 // Few rows per expert: grid (ceil(N / 16), E), NW waves.  A workgroup owns 16 weight rows of one expert; its waves take the
-// width's 32-element steps in turn (weights streamed once, straight into registers), multiply them with up to 16 MT rows of
+// width's 64-element steps in turn (weights streamed once, straight into registers), multiply them with up to 16 MT rows of
 // the segment per pass, and their sums meet in LDS.  K % 32 == 0.
 template <int MT, int NW>
 __global__ __launch_bounds__(64 * NW) void expert_stream_kernel(ExpertArgs a) {
