@@ -1,5 +1,5 @@
 // Causal softmax attention for prompt rows (bf16): one workgroup per (128 consecutive rows of a sequence's run, query head),
-// grouped key / value heads over the paged token-major cache.  Same contract as window_attention.hip's kernels for a window
+// grouped key / value heads over the paged token-major cache.  Same arguments as window_attention.hip's kernels for a window
 // that never ends; optional sink, soft cap, per-key score factor and output gate (per head or per column).
 //
 // Four waves of 32 rows each; keys walk in tiles of 64 up to the last row's own position.  A tile's rows go from the cache to

@@ -1,5 +1,5 @@
 // Causal softmax attention for single rows (decode steps, bf16): one workgroup per (row, key / value head, range of keys), the
-// query heads of the group together, so a cached row is read once.  Same contract as window_attention.hip's kernels for a
+// query heads of the group together, so a cached row is read once.  Same arguments as window_attention.hip's kernels for a
 // window that never ends; optional sink, soft cap, per-key score factor and output gate (per head or per column).
 //
 // Four waves, 32 keys per wave and step.  A step's key and value rows go to the wave's own LDS by direct loads (KEYV: the
